@@ -12,7 +12,7 @@ Per run:
   k_pool / v_pool [pages, ceil(page / pool), kv heads, D | Dv]  fp32 block means; block b sits
       beside the page of its first token b*pool, at entry (b*pool mod page) // pool
   conv [slots, taps - 1, channels]                              the convolution's last inputs
-  ssm  [slots, heads, N, vdim] fp32                             the state-space / delta-rule matrix
+  ssm  [slots, heads, N, vdim] fp32                             the state-space / delta-rule / linear-attention matrix
   lat  [pages, page, 1, kv_rank + R]                            latent attention: normed latent | rotated
       shared key part; a layer that reads another layer's cache holds the same tensor as that run
   canon1 / canon2 [slots, taps - 1, width] fp32                 last inputs of the sublayers' input convolutions
@@ -69,6 +69,8 @@ class PagedCache:
                     d = delta
                     rc.conv = torch.zeros(slots, max(d.conv - 1, 1), d.conv_channels, dtype=dtype, device=device)
                     rc.ssm = torch.zeros(slots, d.heads, d.dim, d.vdim, dtype=torch.float32, device=device)
+                elif getattr(s, "gla", None) is not None:
+                    rc.ssm = torch.zeros(slots, s.gla.heads, s.gla.dim, s.gla.vdim, dtype=torch.float32, device=device)
                 if canon_taps:
                     rc.canon1 = torch.zeros(slots, max(canon_taps - 1, 1), width, dtype=torch.float32, device=device)
                     if getattr(s, "moe", None) is not None or getattr(s, "ff", None):

@@ -109,6 +109,8 @@ class RaggedEngine:
                                 width=cfg.hidden_size, canon_taps=cfg.canon_taps, prev_token=bool(cfg.bigram),
                                 run_layers=[i for i, _ in model.runs])
         self.live: Dict[object, int] = {}
+        # a table of learned positions ends somewhere; every other design's sequences may fill the page pool
+        self.max_positions = cfg.max_position_embeddings if cfg.pos_emb == "learned" else 1 << 30
         # decode-only steps (every sequence brings one token) replay a HIP graph per batch size
         self.use_graphs = (self.device.type == "cuda" and ops.gpu_path(model.embed)) if use_graphs is None \
             else bool(use_graphs)
@@ -137,6 +139,10 @@ class RaggedEngine:
              taps: Optional[list] = None) -> torch.Tensor:
         """``entries``: (request id, its next tokens, indices among them whose logits are wanted).
         A request not yet live is opened.  Returns fp32 logits [wanted rows, vocab] in entry order."""
+        for rid, toks, _ in entries:
+            held = self.length(rid) if rid in self.live else 0
+            if held + len(toks) > self.max_positions:
+                raise ValueError(f"request {rid!r}: {held + len(toks)} tokens, the model has {self.max_positions} positions")
         seqs, ids, rows, off = [], [], [], 0
         for rid, toks, want in entries:
             if len(toks) == 0:
@@ -214,7 +220,7 @@ class RaggedScheduler:
 
     def can_admit(self, prompt_len: int, max_new: int) -> bool:
         c = self.eng.cache
-        return bool(self.free_slots()) and \
+        return bool(self.free_slots()) and prompt_len + max_new <= self.eng.max_positions and \
             c.pages_for(prompt_len + max_new) + self.reserved <= c.num_pages
 
     def admit(self, ids: Sequence[int], max_new: int, eos: Optional[int] = None, tag=None) -> int:
@@ -306,7 +312,7 @@ class RaggedGenerator:
     def __init__(self, model, max_batch: int = 4, max_seq: int = 2048, max_tokens: Optional[int] = None,
                  page: int = 64, prefill_chunk: int = 512):
         self.model, self.cfg, self.device = model, model.cfg, model.device
-        self.max_seq = int(max_seq)
+        self.max_seq = min(int(max_seq), model.cfg.max_position_embeddings)
         tokens = int(max_tokens) if max_tokens else max_batch * ((self.max_seq + page - 1) // page) * page
         self.engine = RaggedEngine(model, tokens, slots=max_batch, page=page)
         self.kv = self.engine.cache

@@ -17,7 +17,9 @@ Families (dims are public HF configs):
                            with one decay per head, sigmoid-routed experts, norms on both sides of
                            every sublayer) and Fikupel (latent attention without positions and gated
                            grouped-query attention with rotated values, both with a window and a sink,
-                           PolyNorm and mixture-of-experts feed-forwards, several residual streams)
+                           PolyNorm and mixture-of-experts feed-forwards, several residual streams) and
+                           Numizen (gated latent attention and gated linear attention beside a gelu-gated
+                           or group-limited expert feed-forward, Dynamic Tanh norms, learned positions)
 A single ``ModelConfig`` describes all decoder families; ``DecoderLM`` interprets the flags.
 """
 from __future__ import annotations
@@ -101,6 +103,7 @@ class LatentAttnSpec:
     rot_scaling: Optional[dict] = None
     kv_from: Optional[int] = None
     sink: bool = False           # exp(sink_h), a learned number per head, joins the softmax denominator
+    gate: bool = False           # the concatenated heads times sigmoid(W_g h), element by element
 
     @property
     def cache_dim(self) -> int:
@@ -207,6 +210,24 @@ class DeltaSpec:
 
 
 @dataclass
+class GLASpec:
+    """Gated linear attention: a [dim, vdim] fp32 state per head that decays by its own factor per key
+    channel and token, S <- diag(a) S + k v^T, o = S^T q, with q scaled by dim^-1/2 and
+    a = sigmoid(W_a2 W_a1 h + b)^(1 / tau) through a projection of rank ``decay_rank``; an RMS norm per head
+    with one weight vector shared by the heads, times silu(W_g h)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    decay_rank: int
+
+    @property
+    def in_sizes(self):
+        """Row blocks of the fused input projection: q | k | v | gate | decay down."""
+        return (self.heads * self.dim, self.heads * self.dim, self.heads * self.vdim, self.heads * self.vdim, self.decay_rank)
+
+
+@dataclass
 class MoESpec:
     """Mixture of gated-linear experts.  ``router`` "softmax": softmax over ``experts``, the ``top``
     largest renormalised and multiplied by ``scale``; "sigmoid": scores sigmoid(W_r h), the ``top``
@@ -214,7 +235,11 @@ class MoESpec:
     softmax over the chosen ones only.  ``act`` "glu_clamp": g = min(W_g h, limit), u = clamp(W_u h, +-limit),
     W_d (g sigmoid(1.702 g) (u + 1)); "silu_glu": W_d (silu(W_g h) (W_u h)).  ``weight_on`` "output":
     the result is sum_k w_k expert_k(h); "input": sum_k expert_k(w_k h).  An optional shared expert of
-    width ``shared_ff`` runs for every token."""
+    width ``shared_ff`` runs for every token, times sigmoid(W_sg h) (one number per token) with ``shared_gate``.
+    ``act`` "relu2" is the unit without a gate, W_d max(W_u h, 0)^2.  Router "softmax" with ``correction``: the
+    experts are chosen by score + correction (a number per expert) and weighted by the score alone; with
+    ``groups`` > 1 equal groups of neighbouring experts: only the ``groups_keep`` groups whose best expert is
+    best can be chosen from."""
     experts: int
     top: int
     scale: float
@@ -226,6 +251,14 @@ class MoESpec:
     act: str = "glu_clamp"
     weight_on: str = "output"
     router_bias: bool = False
+    correction: bool = False
+    groups: int = 1
+    groups_keep: int = 1
+    shared_gate: bool = False
+
+    @property
+    def glu(self) -> bool:
+        return self.act != "relu2"
 
 
 @dataclass
@@ -237,22 +270,26 @@ class LayerSpec:
                                              # "chunk_attention" / "head_delta": one mixer, norms on both sides of each sublayer
                                              # "gated_attention" (and "latent_attention" in a model with ``streams``):
                                              # one mixer, a norm before each sublayer, several residual streams
+                                             # "gla" (and "latent_attention" in a model whose mixer and feed-forward run
+                                             # side by side behind their own norms)
     attn: Optional[WindowAttnSpec] = None
     ssd: Optional[SSDSpec] = None
     ff: Optional[int] = None
     ff_act: str = "relu2"                    # "relu2" | "polynorm" (a N(z) + b N(z^2) + c N(z^3) + e, N = divide by the row's rms)
+                                             # | "gelu_glu" (gelu(W_g h) (W_u h), tanh form)
     latent: Optional[LatentAttnSpec] = None
     delta: Optional[DeltaSpec] = None
     moe: Optional[MoESpec] = None
     chunk_attn: Optional[ChunkAttnSpec] = None
     gated_attn: Optional[GatedAttnSpec] = None
+    gla: Optional[GLASpec] = None
 
 
 @dataclass
 class LoopSpec:
     """Layers [start, stop) run ``times`` times in a row with the same weights.  ``entry``: what
-    happens to the stream right before each pass but the first: "project" (W_in [x ; x0] + step[t])
-    or "add_embed" (x + x0), x0 being the embedding output."""
+    happens to the stream right before each pass but the first: "project" (W_in [x ; x0] + step[t]),
+    "add_embed" (x + x0), x0 being the embedding output, or "plain" (nothing)."""
     start: int
     stop: int
     times: int
@@ -306,6 +343,11 @@ class ModelConfig:
     # own multiple of the sublayer's output); ``hyper`` False: one stream with the plain residual sum
     streams: int = 0
     hyper: bool = True
+    # arch "numizen": ``parallel_residual`` without ``shared_input_norm`` (mixer and feed-forward read their own
+    # norm of the same stream), ``norm`` "dyt" (tanh(alpha x) w + b), ``pos_emb`` "learned" (a row per position
+    # is added to the embedding; no sequence may grow past ``max_position_embeddings``), ``layer_scale`` (each
+    # sublayer's result times a vector before the sum)
+    layer_scale: bool = False
 
     def layer_runs(self) -> List[tuple]:
         """[(layer index, pass number or None)] in execution order; every run has its own cache."""
@@ -490,7 +532,7 @@ def checkpoint_shapes(path: str) -> dict:
 def from_hf_dir(path: str) -> ModelConfig:
     with open(os.path.join(path, "config.json")) as f:
         c = json.load(f)
-    needs_shapes = str(c.get("architecture", "")).lower() in ("pagonex", "fikupel")
+    needs_shapes = str(c.get("architecture", "")).lower() in ("pagonex", "fikupel", "numizen")
     return from_hf_config(c, checkpoint_shapes(path) if needs_shapes else None)
 
 
@@ -822,6 +864,87 @@ def to_fikupel_config(cfg: ModelConfig) -> dict:
     return out
 
 
+def from_numizen_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
+    """The Numizen layout of ``config.json``: ``layers`` (``type`` = ``latent_attention`` or ``gla``, ``mixer``
+    sizes and constants, ``mlp`` = dense, mixture of experts or null), ``loop``, ``max_positions``, ``norm.eps``,
+    ``vocab``, ``width``.  ``shapes`` (tensor name -> shape of the checkpoint) supplies the rank of the linear
+    attention's decay projection and tells which optional tensors are there."""
+    has = (lambda name: name in shapes) if shapes is not None else (lambda name: True)
+    specs = []
+    for i, l in enumerate(c["layers"]):
+        m, kind = l["mixer"], l["type"]
+        lat = gl = None
+        if kind == "latent_attention":
+            rot = m.get("rot") or None
+            lat = LatentAttnSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                                 q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
+                                 rot_dims=int(rot.get("dims", m["rot_dim"])) if rot else 0,
+                                 rot_base=float(rot["base"]) if rot else 10000.0, gate=has(f"l{i}.mix.g"))
+            if lat.rot_dims % 2 or lat.rot_dims > lat.rot_dim:
+                raise ValueError("rotation runs over pairs of coordinates inside the rotated part")
+        elif kind == "gla":
+            rank = int(shapes[f"l{i}.mix.a1"][0]) if shapes is not None else int(m.get("decay_rank", 16))
+            gl = GLASpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), tau=float(m["tau"]), decay_rank=rank)
+        else:
+            raise ValueError(f"unsupported layer type {kind!r}")
+        mlp, moe, ff = l.get("mlp") or None, None, None
+        if mlp and mlp.get("kind", "dense") == "dense":
+            ff = int(mlp["ff"])
+        elif mlp and mlp.get("kind") == "moe":
+            r, sh, g = mlp["router"], mlp.get("shared") or None, mlp["router"].get("groups") or {}
+            moe = MoESpec(experts=int(r["experts"]), top=int(r["top"]), scale=1.0, ff=int(mlp["expert"]["ff"]),
+                          shared_ff=int(sh["ff"]) if sh else 0, router="softmax", act="relu2", weight_on="output",
+                          correction=has(f"l{i}.mlp.correction"), groups=int(g.get("count", 1)),
+                          groups_keep=int(g.get("keep", 1)), shared_gate=bool(sh) and has(f"l{i}.mlp.shared.sg"))
+            if moe.experts % moe.groups or not 1 <= moe.groups_keep <= moe.groups:
+                raise ValueError("the experts must split into equal groups of which at least one is kept")
+            if not 1 <= moe.top <= moe.experts // moe.groups * moe.groups_keep:
+                raise ValueError("the kept groups hold fewer experts than a token uses")
+        elif mlp:
+            raise ValueError(f"unsupported feed-forward kind {mlp.get('kind')!r}")
+        specs.append(LayerSpec("latent_attention" if lat else "gla", ff=ff, ff_act="gelu_glu", latent=lat, moe=moe, gla=gl))
+    lp = c.get("loop") or None
+    if lp and not (0 <= int(lp["start"]) < int(lp["stop"]) <= len(specs) and int(lp["times"]) >= 1):
+        raise ValueError("loop: 0 <= start < stop <= layers and times >= 1")
+    first = specs[0].latent or specs[0].gla
+    return ModelConfig(arch="numizen", vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), num_layers=len(specs),
+                       num_heads=first.heads, num_kv_heads=1, intermediate_size=specs[0].ff or 0, head_dim=first.dim,
+                       max_position_embeddings=int(shapes["pos"][0]) if shapes is not None else int(c["max_positions"]),
+                       norm="dyt", norm_eps=float(c["norm"]["eps"]), act="gelu_tanh", parallel_residual=True,
+                       pos_emb="learned", name=c.get("name", "numizen"), layer_specs=specs,
+                       loop=LoopSpec(int(lp["start"]), int(lp["stop"]), int(lp["times"]), "plain") if lp else None,
+                       layer_scale=has("l0.ls1"))
+
+
+def to_numizen_config(cfg: ModelConfig) -> dict:
+    """Inverse of ``from_numizen_config`` (the decay ranks travel as tensor shapes)."""
+    layers = []
+    for s in cfg.layer_specs:
+        if s.latent is not None:
+            a = s.latent
+            m = {"heads": a.heads, "dim": a.dim, "rot_dim": a.rot_dim, "vdim": a.vdim, "q_rank": a.q_rank,
+                 "kv_rank": a.kv_rank, "scale": a.scale}
+            if a.rot_dims:
+                m["rot"] = {"dims": a.rot_dims, "base": a.rot_base}
+        else:
+            m = {"heads": s.gla.heads, "dim": s.gla.dim, "vdim": s.gla.vdim, "tau": s.gla.tau}
+        mlp = None
+        if s.moe is not None:
+            e = s.moe
+            mlp = {"kind": "moe", "router": {"experts": e.experts, "top": e.top, "groups": {"count": e.groups, "keep": e.groups_keep}},
+                   "expert": {"ff": e.ff}}
+            if e.shared_ff:
+                mlp["shared"] = {"ff": e.shared_ff}
+        elif s.ff:
+            mlp = {"kind": "dense", "ff": s.ff}
+        layers.append({"type": s.mixer, "mixer": m, "mlp": mlp})
+    out = {"architecture": "Numizen", "vocab": cfg.vocab_size, "width": cfg.hidden_size, "layers": layers,
+           "norm": {"eps": cfg.norm_eps}, "max_positions": cfg.max_position_embeddings}
+    if cfg.loop is not None:
+        out["loop"] = {"start": cfg.loop.start, "stop": cfg.loop.stop, "times": cfg.loop.times}
+    return out
+
+
 def from_hf_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
     """Map a ``config.json`` onto ModelConfig (Hugging Face ``model_type`` layouts, or an
     ``architecture`` key naming a per-layer layout; ``shapes``: the checkpoint's tensor shapes, for
@@ -834,6 +957,8 @@ def from_hf_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
         return from_vetevik_config(c)
     if str(c.get("architecture", "")).lower() == "fikupel":
         return from_fikupel_config(c, shapes)
+    if str(c.get("architecture", "")).lower() == "numizen":
+        return from_numizen_config(c, shapes)
     mt = c.get("model_type")
     eos = c.get("eos_token_id")
     if isinstance(eos, list):

@@ -1,6 +1,6 @@
-"""Layer-spec language models (arch "nudadra", "pagonex", "vetevik", "fikupel"): every layer is described by its own
-entry of ``ModelConfig.layer_specs``, a span of layers may run several times in a row, and the
-residual stream is fp32.
+"""Layer-spec language models (arch "nudadra", "pagonex", "vetevik", "fikupel", "numizen"): every layer is
+described by its own entry of ``ModelConfig.layer_specs``, a span of layers may run several times in a row,
+and the residual stream is fp32.
 
 Per layer (post-norm form, ``PostNormLayer``):  x <- x + LN1(mixer(x + conv1(x))) ;
 x <- x + LN2(ff(x + conv2(x))): the sublayers read the stream itself plus a causal depthwise
@@ -21,6 +21,11 @@ u = sum_s a_s x_s, computes y = f(RMSnorm(u)), and every stream becomes x_r <- s
 mixer is latent attention without positions or gated grouped-query attention, the feed-forward a
 PolyNorm unit or a mixture of experts; the final norm reads the sum of the streams and the embedding
 table is the output projection.
+
+Per layer (side by side behind two norms, ``TwoNormLayer``):  x <- x + s1 mixer(N1(x)) + s2 ff(N2(x)), both of the
+same x, every N a Dynamic Tanh (tanh(alpha x) w + b) and s1, s2 learned vectors.  The mixer is latent attention
+with an output gate or gated linear attention, the feed-forward a gelu-gated unit or a mixture of squared-ReLU
+experts.  The embedding adds a learned row per position; nothing happens between the passes of a looped span.
 
 Per layer (parallel form):  h = norm(x) ;  x <- x + mixer(h) + ff(h), with one norm whose gain is a
 single number, a ``ParallelMixer`` (models/mixers.py) and a squared-ReLU feed-forward.  The
@@ -45,10 +50,10 @@ import torch.nn as nn
 
 from ..ops import seqmix
 from .configs import LayerSpec, ModelConfig
-from .layers import GroupRMSNorm, Linear, RowLayerNorm, ScalarNorm
-from .mixers import (ChannelDeltaMixer, ChunkAttention, GatedAttention, HeadDeltaMixer, LatentAttention,
-                     ParallelMixer)
-from .moe import MoEFeedForward
+from .layers import DynamicTanh, GroupRMSNorm, Linear, RowLayerNorm, ScalarNorm
+from .mixers import (ChannelDeltaMixer, ChunkAttention, GatedAttention, GatedLinearAttention, HeadDeltaMixer,
+                     LatentAttention, ParallelMixer)
+from .moe import MoEFeedForward, MoEOut
 
 
 class HybridLayer(nn.Module):
@@ -235,9 +240,67 @@ class HyperLayer(nn.Module):
         return X, None
 
 
+class GeluGLUFF(nn.Module):
+    """W_down (gelu(W_gate h) (W_up h)), tanh form of gelu; gate and up rows are one GEMM."""
+
+    def __init__(self, width: int, ff: int, dtype, device):
+        super().__init__()
+        self.ff = ff
+        self.gate_up = Linear(width, 2 * ff, False, dtype, device)
+        self.down = Linear(ff, width, False, dtype, device)
+
+    def run(self, h: torch.Tensor) -> MoEOut:
+        return MoEOut(self.down(seqmix.glu_gelu(self.gate_up(h), self.ff)), None, None, None, None)
+
+
+class TwoNormLayer(nn.Module):
+    """One mixer (gated latent attention or gated linear attention) and an optional feed-forward side by side on
+    their own Dynamic Tanh norms of the same stream, each result times a learned vector before the sum."""
+
+    def __init__(self, cfg: ModelConfig, spec: LayerSpec, idx: int, dtype, device):
+        super().__init__()
+        W, eps = cfg.hidden_size, cfg.norm_eps
+        self.idx, self.spec, self.dtype = idx, spec, dtype
+        if spec.mixer == "latent_attention":
+            self.mix = LatentAttention(spec.latent, W, eps, dtype, device)
+        elif spec.mixer == "gla":
+            self.mix = GatedLinearAttention(spec.gla, W, eps, dtype, device)
+        else:
+            raise ValueError(spec.mixer)
+        if spec.moe is not None:
+            self.ff = MoEFeedForward(spec.moe, W, dtype, device)
+        elif spec.ff:
+            assert spec.ff_act == "gelu_glu", spec.ff_act
+            self.ff = GeluGLUFF(W, spec.ff, dtype, device)
+        else:
+            self.ff = None
+        S = lambda: nn.Parameter(torch.ones(W, dtype=torch.float32, device=device), requires_grad=False) \
+            if cfg.layer_scale else None
+        self.norm1, self.ls1 = DynamicTanh(W, device), S()
+        if self.ff is not None:
+            self.norm2, self.ls2 = DynamicTanh(W, device), S()
+
+    def norms(self) -> tuple:
+        """What this layer reads of the stream: the layer before computes it while it adds its own results."""
+        return (self.norm1.params, self.norm2.params) if self.ff is not None else (self.norm1.params,)
+
+    def forward(self, x: torch.Tensor, meta: seqmix.RaggedMeta, run, h: Optional[tuple] = None, nxt: Optional[tuple] = None):
+        """``h``: this layer's normed inputs when the layer before already computed them; ``nxt``: the next
+        layer's ``norms()``.  Returns (x updated in place, the next layer's normed inputs or None)."""
+        if h is None:
+            h = seqmix.parallel_update(x, self.norms(), self.dtype)
+        m = self.mix(h[0], meta, run)
+        f = self.ff.run(h[1]) if self.ff is not None else MoEOut(None, None, None, None, None)
+        out = seqmix.parallel_update(x, nxt or (), self.dtype, m, self.ls1, f.shared, f.shared_w, f.parts, f.wts, f.rows,
+                                     self.ls2 if self.ff is not None else None)
+        return x, (out if nxt is not None else None)
+
+
 def _make_layer(cfg: ModelConfig, spec: LayerSpec, idx: int, dtype, device) -> nn.Module:
     if cfg.streams:
         return HyperLayer(cfg, spec, idx, dtype, device)
+    if cfg.parallel_residual and not cfg.shared_input_norm:
+        return TwoNormLayer(cfg, spec, idx, dtype, device)
     if spec.mixer == "parallel":
         return HybridLayer(cfg, spec, idx, dtype, device)
     if spec.mixer in ("chunk_attention", "head_delta"):
@@ -258,6 +321,8 @@ class HybridLM(nn.Module):
         self.embed = nn.Parameter(torch.empty(cfg.vocab_size, W, dtype=dtype, device=device), requires_grad=False)
         self.layers = nn.ModuleList([_make_layer(cfg, s, i, dtype, device) for i, s in enumerate(cfg.layer_specs)])
         self.runs = cfg.layer_runs()
+        if cfg.pos_emb == "learned":
+            self.pos = nn.Parameter(torch.empty(cfg.max_position_embeddings, W, dtype=dtype, device=device), requires_grad=False)
         if cfg.bigram:
             self.bigram = nn.Parameter(torch.empty(cfg.bigram["buckets"] + 1, W, dtype=dtype, device=device),
                                        requires_grad=False)
@@ -268,6 +333,7 @@ class HybridLM(nn.Module):
         self.final_norm = StreamNorm(W, cfg.norm_eps, device) if cfg.streams else \
             ScalarNorm(cfg.norm_eps, device) if cfg.norm == "rms_scalar" else \
             GroupRMSNorm(W, cfg.norm_groups, cfg.norm_eps, device) if cfg.norm == "rms_group" else \
+            DynamicTanh(W, device) if cfg.norm == "dyt" else \
             RowLayerNorm(W, cfg.norm_eps, device)
         self.lm_head = Linear(W, cfg.vocab_size, False, dtype, device)
         if cfg.tie_word_embeddings:                      # the embedding table is the output projection
@@ -300,20 +366,25 @@ class HybridLM(nn.Module):
             b = cfg.bigram
             x0 = seqmix.embedding_bigram(ids, meta, self.embed, self.bigram, cache.prev_tok, b["buckets"], b["mul_prev"],
                                          b["mul_cur"])
+        elif cfg.pos_emb == "learned":
+            x0 = seqmix.embedding_learned(ids, meta, self.embed, self.pos)
         else:
             x0 = seqmix.embedding_scaled(ids, self.embed, cfg.embed_scale)
-        x = x0.clone() if cfg.loop is not None else x0
+        x = x0.clone() if cfg.loop is not None and cfg.loop.entry != "plain" else x0
         if cfg.streams:                                  # [T, S, W]: every stream starts as the embedding rows
             x = x0[:, None, :].expand(-1, cfg.streams, -1).contiguous()
         h_next = None
         for r, (i, t) in enumerate(self.runs):
-            if t is not None and i == cfg.loop.start:
+            if t is not None and i == cfg.loop.start and cfg.loop.entry != "plain":
                 if cfg.loop.entry == "add_embed":
                     if t > 0:                            # every pass but the first starts from x + the embedding rows
                         x.add_(x0)
                 else:
                     x = seqmix.linear_f32(seqmix.cat_cast(x, x0, self.dtype), self.loop_in.weight, self.loop_step[t])
-            if cfg.streams:                              # the next layer's read + norm rides on this layer's last rebuild
+            if isinstance(self.layers[i], TwoNormLayer):  # the next layer's norms ride on this layer's residual sum
+                nxt = self.layers[self.runs[r + 1][0]].norms() if r + 1 < len(self.runs) else None
+                x, h_next = self.layers[i](x, meta, cache.run(r), h_next, nxt)
+            elif cfg.streams:                            # the next layer's read + norm rides on this layer's last rebuild
                 nxt = self.layers[self.runs[r + 1][0]].first_read() if r + 1 < len(self.runs) and cfg.loop is None else None
                 x, h_next = self.layers[i](x, meta, cache.run(r), h_next, nxt)
             else:
@@ -630,10 +701,104 @@ def export_fikupel_tensors(model: "HybridLM") -> Dict[str, torch.Tensor]:
     return {k: v.to(torch.bfloat16).contiguous() for k, v in out.items()}
 
 
+def _numizen_norm_names(cfg: ModelConfig, i: int, spec: LayerSpec) -> list:
+    """(parameter, checkpoint name) pairs of a layer's norms and scales."""
+    out = []
+    for n in ("1", "2") if spec.moe is not None or spec.ff else ("1",):
+        out += [(f"layers.{i}.norm{n}.weight", f"l{i}.norm{n}"), (f"layers.{i}.norm{n}.bias", f"l{i}.norm{n}.b"),
+                (f"layers.{i}.norm{n}.alpha", f"l{i}.norm{n}.alpha")]
+        if cfg.layer_scale:
+            out.append((f"layers.{i}.ls{n}", f"l{i}.ls{n}"))
+    return out
+
+
+_NUMIZEN_TOP = [("embed", "embed"), ("pos", "pos"), ("final_norm.weight", "final.norm"), ("final_norm.bias", "final.norm.b"),
+                ("final_norm.alpha", "final.norm.alpha"), ("lm_head.weight", "head")]
+
+
+def convert_numizen_tensors(cfg: ModelConfig, t: Dict[str, torch.Tensor]) -> Dict[str, torch.Tensor]:
+    """Checkpoint names of the Numizen layout (``l<i>.norm1.alpha``, ``l<i>.mix.dq``, ``l<i>.mlp.e<k>.up`` ...) ->
+    this package's parameter names: fused input projections, per-head key / value expansions, stacked expert
+    weights, the shared expert's gate as the router's last row."""
+    out = {ours: t[theirs] for ours, theirs in _NUMIZEN_TOP}
+    for i, spec in enumerate(cfg.layer_specs):
+        out.update({ours: t[theirs] for ours, theirs in _numizen_norm_names(cfg, i, spec)})
+        M, m = f"l{i}.mix.", f"layers.{i}.mix."
+        if spec.latent is not None:
+            a = spec.latent
+            out[m + "proj_in.weight"] = torch.cat([t[M + n] for n in ("dq", "dkv") + (("g",) if a.gate else ())], 0)
+            out[m + "q_norm"], out[m + "kv_norm"] = t[M + "dq.norm"], t[M + "dkv.norm"]
+            out[m + "uq.weight"] = t[M + "uq"]
+            out[m + "uk"] = t[M + "uk"].reshape(a.heads, a.dim, a.kv_rank)
+            out[m + "uv"] = t[M + "uv"].reshape(a.heads, a.vdim, a.kv_rank).transpose(1, 2).contiguous()
+        else:
+            out[m + "proj_in.weight"] = torch.cat([t[M + n] for n in ("q", "k", "v", "g", "a1")], 0)
+            out[m + "a2"], out[m + "a2_b"], out[m + "norm_w"] = t[M + "a2"], t[M + "a2.b"], t[M + "norm"]
+        out[m + "o.weight"] = t[M + "o"]
+        F_, f = f"l{i}.mlp.", f"layers.{i}.ff."
+        if spec.moe is not None:
+            e = spec.moe
+            out[f + "router"] = torch.cat([t[F_ + "router"]] + ([t[F_ + "shared.sg"]] if e.shared_gate else []), 0)
+            if e.correction:
+                out[f + "correction"] = t[F_ + "correction"]
+            out[f + "w_gu"] = torch.stack([t[f"{F_}e{k}.up"] for k in range(e.experts)])
+            out[f + "w_down"] = torch.stack([t[f"{F_}e{k}.down"] for k in range(e.experts)])
+            if e.shared_ff:
+                out[f + "shared_gu.weight"], out[f + "shared_down.weight"] = t[F_ + "shared.up"], t[F_ + "shared.down"]
+        elif spec.ff:
+            out[f + "gate_up.weight"] = torch.cat([t[F_ + "gate"], t[F_ + "up"]], 0)
+            out[f + "down.weight"] = t[F_ + "down"]
+    return out
+
+
+def export_numizen_tensors(model: "HybridLM") -> Dict[str, torch.Tensor]:
+    """Inverse of ``convert_numizen_tensors`` (checkpoint names, 16-bit storage)."""
+    cfg = model.cfg
+    p = {k: v.detach() for k, v in model.named_parameters()}
+    out = {theirs: p[ours] for ours, theirs in _NUMIZEN_TOP}
+    for i, spec in enumerate(cfg.layer_specs):
+        out.update({theirs: p[ours] for ours, theirs in _numizen_norm_names(cfg, i, spec)})
+        M, m = f"l{i}.mix.", f"layers.{i}.mix."
+        w = p[m + "proj_in.weight"]
+        if spec.latent is not None:
+            a = spec.latent
+            cut = a.q_rank + a.cache_dim
+            out[M + "dq"], out[M + "dkv"] = w[:a.q_rank], w[a.q_rank:cut]
+            if a.gate:
+                out[M + "g"] = w[cut:]
+            out[M + "dq.norm"], out[M + "dkv.norm"] = p[m + "q_norm"], p[m + "kv_norm"]
+            out[M + "uq"] = p[m + "uq.weight"]
+            out[M + "uk"] = p[m + "uk"].reshape(a.heads * a.dim, a.kv_rank)
+            out[M + "uv"] = p[m + "uv"].transpose(1, 2).reshape(a.heads * a.vdim, a.kv_rank)
+        else:
+            for n, part in zip(("q", "k", "v", "g", "a1"), torch.split(w, list(spec.gla.in_sizes), 0)):
+                out[M + n] = part
+            out[M + "a2"], out[M + "a2.b"], out[M + "norm"] = p[m + "a2"], p[m + "a2_b"], p[m + "norm_w"]
+        out[M + "o"] = p[m + "o.weight"]
+        F_, f = f"l{i}.mlp.", f"layers.{i}.ff."
+        if spec.moe is not None:
+            e = spec.moe
+            out[F_ + "router"] = p[f + "router"][:e.experts]
+            if e.shared_gate:
+                out[F_ + "shared.sg"] = p[f + "router"][e.experts:]
+            if e.correction:
+                out[F_ + "correction"] = p[f + "correction"]
+            for k in range(e.experts):
+                out[f"{F_}e{k}.up"], out[f"{F_}e{k}.down"] = p[f + "w_gu"][k], p[f + "w_down"][k]
+            if e.shared_ff:
+                out[F_ + "shared.up"], out[F_ + "shared.down"] = p[f + "shared_gu.weight"], p[f + "shared_down.weight"]
+        elif spec.ff:
+            out[F_ + "gate"], out[F_ + "up"] = p[f + "gate_up.weight"][:spec.ff], p[f + "gate_up.weight"][spec.ff:]
+            out[F_ + "down"] = p[f + "down.weight"]
+    out = {k: v.to(torch.bfloat16).contiguous() for k, v in out.items()}
+    return {k: v.reshape(()) if k.endswith(".alpha") else v for k, v in out.items()}
+
+
 CONVERTERS = {"nudadra": (convert_nudadra_tensors, export_nudadra_tensors),
               "pagonex": (convert_pagonex_tensors, export_pagonex_tensors),
               "vetevik": (convert_vetevik_tensors, export_vetevik_tensors),
-              "fikupel": (convert_fikupel_tensors, export_fikupel_tensors)}
+              "fikupel": (convert_fikupel_tensors, export_fikupel_tensors),
+              "numizen": (convert_numizen_tensors, export_numizen_tensors)}
 
 
 @torch.no_grad()
@@ -644,6 +809,8 @@ def load_into_hybrid(model: HybridLM, tensors: Dict[str, torch.Tensor]) -> Hybri
         if t is None:
             missing.append(name)
             continue
+        if t.dim() == 0:                                 # a single number is stored without an axis
+            t = t.reshape(1)
         assert tuple(t.shape) == tuple(p.shape), f"{name}: {tuple(t.shape)} vs {tuple(p.shape)}"
         p.copy_(t.to(p.dtype))
     if missing:
@@ -689,6 +856,18 @@ def init_random_hybrid_(model: HybridLM, seed: int = 0) -> HybridLM:
             v = 1.0 + 0.1 * r(*p.shape)
         elif leaf == "act":
             v = torch.tensor([1.0, 0.5, 0.25, 0.0]) + 0.1 * r(*p.shape)
+        elif leaf == "alpha":
+            v = 0.5 + 0.1 * r(*p.shape)
+        elif name == "pos":
+            v = 0.3 * r(*p.shape)
+        elif leaf in ("ls1", "ls2"):
+            v = 0.5 + 0.1 * r(*p.shape)
+        elif leaf == "a2":
+            v = r(*p.shape) / p.shape[1] ** 0.5
+        elif leaf == "a2_b":                             # decays that keep a token for tens to hundreds of steps
+            v = 2.0 + r(*p.shape)
+        elif leaf == "correction":
+            v = 0.02 * r(*p.shape)
         elif leaf == "router_b":
             v = 0.5 * r(*p.shape)
         elif leaf == "sink":

@@ -306,6 +306,24 @@ class GroupRMSNorm(nn.Module):
         return ops.seqmix.group_norm_residual(x, y, self.weight, self.groups, self.eps, mult, parts, part_w)
 
 
+class DynamicTanh(nn.Module):
+    """tanh(alpha x) weight + bias with one learned number alpha, no statistics, over fp32 rows (the residual
+    stream of the layer-spec models), rows of the consumer's dtype out."""
+
+    def __init__(self, width: int, device=None):
+        super().__init__()
+        self.weight = nn.Parameter(torch.ones(width, dtype=torch.float32, device=device), requires_grad=False)
+        self.bias = nn.Parameter(torch.zeros(width, dtype=torch.float32, device=device), requires_grad=False)
+        self.alpha = nn.Parameter(torch.ones(1, dtype=torch.float32, device=device), requires_grad=False)
+
+    @property
+    def params(self):
+        return self.weight, self.bias, self.alpha
+
+    def forward(self, x: torch.Tensor, out_dtype=torch.bfloat16) -> torch.Tensor:
+        return ops.seqmix.parallel_update(x, (self.params,), out_dtype)[0]
+
+
 def act_fn(x, act: str, quant: bool):
     if quant:
         q, s = ops.activation_quant(x, act)

@@ -16,7 +16,7 @@ import torch
 import torch.nn as nn
 
 from ..ops import seqmix
-from .configs import ChunkAttnSpec, DeltaSpec, GatedAttnSpec, SSDSpec, WindowAttnSpec
+from .configs import ChunkAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, SSDSpec, WindowAttnSpec
 from .layers import Linear
 
 
@@ -153,7 +153,8 @@ class LatentAttention(nn.Module):
     latent as the value; each head's weighted latent is then expanded by W_uv,h.  The cache is read
     once for all heads and nothing per head is stored.  A layer with ``kv_from`` reads another
     layer's cached rows and has no down projection of its own.  ``rot_dim`` 0: no rotated part at all
-    (attention without positions); ``sink``: a learned number per head in the softmax denominator."""
+    (attention without positions); ``sink``: a learned number per head in the softmax denominator; ``gate``: the
+    concatenated heads times sigmoid(W_g h), element by element."""
 
     def __init__(self, spec, width: int, eps: float, dtype, device):
         super().__init__()
@@ -161,8 +162,9 @@ class LatentAttention(nn.Module):
         s = spec
         P = lambda *shape: nn.Parameter(torch.zeros(*shape, dtype=torch.float32, device=device), requires_grad=False)
         self.own_kv = s.kv_from is None
-        # rows: query latent | (key / value latent | shared key part)
-        self.proj_in = Linear(width, s.q_rank + (s.cache_dim if self.own_kv else 0), False, dtype, device)
+        # rows: query latent | (key / value latent | shared key part) | output gate
+        self.ng = s.heads * s.vdim if s.gate else 0
+        self.proj_in = Linear(width, s.q_rank + (s.cache_dim if self.own_kv else 0) + self.ng, False, dtype, device)
         self.q_norm = P(s.q_rank)
         self.kv_norm = P(s.kv_rank) if self.own_kv else None
         self.uq = Linear(s.q_rank, s.heads * (s.dim + s.rot_dim), False, dtype, device)
@@ -178,14 +180,16 @@ class LatentAttention(nn.Module):
         u = self.proj_in(h)
         cq = seqmix.rms_norm_cols(u, 0, s.q_rank, self.q_norm, self.eps, h.dtype)
         q = self.uq(cq).view(T, H, s.dim + s.rot_dim)
-        q_lat = torch.bmm(q[:, :, :s.dim].transpose(0, 1), self.uk).transpose(0, 1)      # [T, H, kv_rank]
         rope = _shared_rope(self._rope, (s.rot_dims, s.rot_base, s.rot_scaling), meta.max_keys, h.device)
-        qc = seqmix.latent_write(u if self.own_kv else None, s.q_rank, self.kv_norm, self.eps, q, q_lat, meta, rope,
-                                 run.lat, s.kv_rank, s.rot_dims)
+        if self.own_kv:
+            qc = seqmix.latent_expand_write(u, s.q_rank, self.kv_norm, self.eps, q, self.uk, meta, rope, run.lat, s.kv_rank,
+                                            s.rot_dims)
+        else:
+            q_lat = torch.bmm(q[:, :, :s.dim].transpose(0, 1), self.uk).transpose(0, 1)  # [T, H, kv_rank]
+            qc = seqmix.latent_write(None, s.q_rank, None, self.eps, q, q_lat, meta, rope, run.lat, s.kv_rank, s.rot_dims)
         a = seqmix.window_pool_attention(qc, None, run.lat, run.lat[..., :s.kv_rank], None, None, meta, s.scale,
                                          s.window, None, self.sink)                     # [T, H * kv_rank]
-        v = torch.bmm(a.view(T, H, s.kv_rank).transpose(0, 1), self.uv).transpose(0, 1)  # [T, H, vdim]
-        return self.o(v.reshape(T, H * s.vdim))
+        return self.o(seqmix.head_expand_gate(a, self.uv, u[:, u.shape[1] - self.ng:] if self.ng else None, meta))
 
 
 class GatedAttention(nn.Module):
@@ -221,6 +225,26 @@ class GatedAttention(nn.Module):
         if vrope is not None or ng:
             a = seqmix.unrotate_gate(a, u[:, nq + nk + nv:nq + nk + nv + ng] if ng else None, meta, vrope, s.heads)
         return self.o(a)
+
+
+class GatedLinearAttention(nn.Module):
+    """Gated linear attention: per head S <- diag(a) S + k v^T and o = S^T q over a [dim, vdim] fp32 state,
+    a = sigmoid(W_a2 W_a1 h + b)^(1 / tau) per key channel, a per-head RMS norm times silu(W_g h), and the
+    output projection.  One fused GEMM produces q | k | v | gate and the decay projection's inner rows."""
+
+    def __init__(self, spec: GLASpec, width: int, eps: float, dtype, device):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        s = spec
+        P = lambda *shape: nn.Parameter(torch.zeros(*shape, dtype=torch.float32, device=device), requires_grad=False)
+        self.proj_in = Linear(width, sum(s.in_sizes), False, dtype, device)
+        self.a2, self.a2_b, self.norm_w = P(s.heads * s.dim, s.decay_rank), P(s.heads * s.dim), P(s.vdim)
+        self.o = Linear(s.heads * s.vdim, width, False, dtype, device)
+
+    def forward(self, h: torch.Tensor, meta: seqmix.RaggedMeta, run) -> torch.Tensor:
+        s = self.spec
+        return self.o(seqmix.gated_linear_attention(self.proj_in(h), self.a2, self.a2_b, self.norm_w, run.ssm, meta, s.heads,
+                                                    s.dim, s.vdim, s.tau, self.eps))
 
 
 class ChannelDeltaMixer(nn.Module):

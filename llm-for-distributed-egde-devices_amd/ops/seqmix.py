@@ -584,6 +584,76 @@ def latent_write(u: Optional[torch.Tensor], c0: int, weight: Optional[torch.Tens
     return torch.cat([q_lat.float(), qr], -1).to(q.dtype)
 
 
+# decode-sized steps carry the queries through the key expansion inside the cache-write kernel and expand the
+# heads' outputs (with their gate) in one kernel; larger steps run batched products around the same kernels
+HEAD_FUSE_MAX = int(__import__("os").environ.get("EDGELLM_HEAD_FUSE_MAX", "16"))
+
+
+def latent_expand_write(u: torch.Tensor, c0: int, weight: torch.Tensor, eps: float, q: torch.Tensor, uk: torch.Tensor,
+                        meta: RaggedMeta, rope: Optional[torch.Tensor], pages: torch.Tensor, kv_rank: int,
+                        rot_dims: int) -> torch.Tensor:
+    """``latent_write`` that also computes q_lat[t, h] = q[t, h, :D] uk[h] (uk [H, D, kv_rank]); on the GPU one
+    kernel at up to HEAD_FUSE_MAX tokens."""
+    D = uk.shape[1]
+    if _gpu(q) and q.shape[0] <= HEAD_FUSE_MAX:
+        return _ext().sm_latent_expand_write(u, int(c0), weight, float(eps), q, uk, meta.tok_seq, meta.tok_pos, meta.seq_slot,
+                                             meta.page_table, rope if rot_dims else None, pages, int(rot_dims))
+    q_lat = torch.bmm(q[:, :, :D].transpose(0, 1), uk).transpose(0, 1)                  # [T, H, kv_rank]
+    return latent_write(u, c0, weight, eps, q, q_lat, meta, rope, pages, kv_rank, rot_dims)
+
+
+def head_expand_gate(a: torch.Tensor, uv: torch.Tensor, gate: Optional[torch.Tensor], meta: RaggedMeta) -> torch.Tensor:
+    """a [T, H * kv_rank] (each head's weighted latent) -> [T, H * Dv]: head h's part times uv[h] (uv
+    [H, kv_rank, Dv]), times sigmoid(gate) element by element (``gate`` [T, H * Dv] view; None: 1)."""
+    T, (H, R, Dv) = a.shape[0], uv.shape
+    if _gpu(a) and T <= HEAD_FUSE_MAX:
+        return _ext().sm_head_expand_gate(a, uv, gate)
+    v = torch.bmm(a.view(T, H, R).transpose(0, 1), uv)                                   # [H, T, Dv]
+    if gate is None:
+        return v.transpose(0, 1).reshape(T, H * Dv)
+    if _gpu(a):
+        return _ext().sm_heads_gate(v, gate)
+    return (v.transpose(0, 1).reshape(T, H * Dv).float() * torch.sigmoid(gate.float())).to(a.dtype)
+
+
+# --------------------------------------------------------------------------- gated linear attention
+GLA_CHUNK_MIN = int(__import__("os").environ.get("EDGELLM_GLA_CHUNK_MIN", "24"))
+
+
+def gated_linear_attention(u: torch.Tensor, a2: torch.Tensor, a2_b: torch.Tensor, norm_w: torch.Tensor, state: torch.Tensor,
+                           meta: RaggedMeta, heads: int, N: int, P: int, tau: float, eps: float) -> torch.Tensor:
+    """u [T, q | k | v | gate | decay down] (a layer's fused input projection) -> [T, heads P] in u's dtype.
+
+    In fp32, per head: log a = log sigmoid(a2 d + a2_b) / tau per key channel (d the decay-down columns, a2
+    [heads N, rank], a2_b fp32 [heads N]); S <- diag(a) S + k v^T; o = S^T q N^-1/2; then o over its root mean
+    square times ``norm_w`` fp32 [P], times silu(gate).  state [slots, heads, N, P] fp32 is read (zero for a
+    portion starting at 0) and left at the portion's end."""
+    HN, HP = heads * N, heads * P
+    if _gpu(u):
+        # portions of GLA_CHUNK_MIN tokens or more: kernels parallel over 64-token chunks; shorter steps (decode):
+        # one workgroup per (sequence, head), token by token, with the decays, the norm and the gate in it
+        chunks = max_chunks = 0
+        if meta.max_len >= GLA_CHUNK_MIN:
+            per = [(h[2] + 63) // 64 for h in meta.host]
+            chunks, max_chunks = sum(per), max(per)
+        return _ext().sm_gla(u, a2, a2_b, norm_w, state, meta.seq_slot, meta.seq_start, meta.seq_len, meta.seq_off,
+                             int(meta.n), int(heads), int(N), int(P), float(tau), float(eps), int(chunks), int(max_chunks))
+    T = u.shape[0]
+    y = torch.empty(T, HP, dtype=torch.float32, device=u.device)
+    z = F.linear(u[:, 2 * HN + 2 * HP:].float(), a2.float(), a2_b.float())
+    a = torch.exp(F.logsigmoid(z) / tau).view(T, heads, N)
+    for slot, start, n, off in meta.host:
+        x = u[off:off + n].float()
+        q, k = x[:, :HN].view(n, heads, N) * N ** -0.5, x[:, HN:2 * HN].view(n, heads, N)
+        v = x[:, 2 * HN:2 * HN + HP].view(n, heads, P)
+        S = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
+        for t in range(n):
+            S = a[off + t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            y[off + t] = torch.einsum("hnp,hn->hp", S, q[t]).reshape(HP)
+        state[slot] = S
+    return head_norm_gate(y, u[:, 2 * HN + HP:2 * HN + 2 * HP], norm_w, heads, eps, u.dtype, act="silu")
+
+
 # --------------------------------------------------------------------------- gated delta rule
 def delta_prepare(qkv: torch.Tensor, u: torch.Tensor, b0: int, a: torch.Tensor, dt_bias: torch.Tensor,
                   A_log: torch.Tensor, heads: int, kv_heads: int, N: int):
@@ -666,6 +736,32 @@ def head_norm_gate(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, heads
 
 
 # --------------------------------------------------------------------------- mixture of experts
+def moe_route_grouped(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, correction: Optional[torch.Tensor],
+                      groups: int = 1, keep: int = 1, gate: bool = False):
+    """Router in fp32 whose choice and weights differ: scores s = softmax(W_r h) over the E experts, choice
+    scores c = s + ``correction`` (fp32 [E] or None).  The experts form ``groups`` equal groups of neighbours;
+    only those of the ``keep`` groups with the largest best c stay open, and the ``top`` open experts with the
+    largest c are chosen (the lower id on a tie).  Their weights are s over the sum of the chosen s (+ 1e-20),
+    times ``scale``.  ``gate``: router has a last row E + 1 whose logit is no expert's; its sigmoid comes back
+    as a third result fp32 [T] (the weight of a shared expert).  Returns (ids int32 [T, top], weights fp32
+    [T, top], gate or None), best choice first."""
+    E = router.shape[0] - int(gate)
+    if _gpu(h):
+        idx, wts, gw = _ext().sm_moe_route_grouped(h, router, correction, int(top), float(scale), int(groups), int(keep),
+                                                   bool(gate))
+        return idx, wts, gw if gate else None
+    z = h.float() @ router.float().t()
+    s = torch.softmax(z[:, :E], -1)
+    c = s if correction is None else s + correction.float()
+    if groups > 1:
+        best = c.view(-1, groups, E // groups).amax(-1)
+        open_ = torch.zeros_like(best, dtype=torch.bool).scatter_(1, torch.sort(best, dim=-1, descending=True, stable=True)[1][:, :keep], True)
+        c = c.masked_fill(~open_.repeat_interleave(E // groups, 1), float("-inf"))
+    idx = torch.sort(c, dim=-1, descending=True, stable=True)[1][:, :top]
+    w = s.gather(1, idx)
+    return idx.int(), w / (w.sum(-1, keepdim=True) + 1e-20) * scale, torch.sigmoid(z[:, E]) if gate else None
+
+
 def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, mode: str = "softmax",
               bias: Optional[torch.Tensor] = None):
     """Router in fp32 over h [T, W] (router fp32 [E, W], logits W_r h + ``bias`` fp32 [E]).  ``mode``
@@ -694,30 +790,45 @@ MOE_GEMM_MIN = int(__import__("os").environ.get("EDGELLM_MOE_GEMM_MIN", "64"))
 
 
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, w_gu: torch.Tensor, w_down: torch.Tensor, limit: float,
-                act: str = "glu_clamp", in_w: Optional[torch.Tensor] = None) -> torch.Tensor:
+                act: str = "glu_clamp", in_w: Optional[torch.Tensor] = None, sorted_rows: bool = False):
     """Every token's chosen experts: h [T, W], idx int32 [T, top], w_gu [E, 2 ff, W] (gate rows, then
     up rows), w_down [E, W, ff] -> the experts' outputs [T, top, W] (not yet weighted).  ``act``
-    "glu_clamp" (with ``limit``) or "silu_glu"; ``in_w`` fp32 [T, top] (silu_glu only): choice k runs on
+    "glu_clamp" (with ``limit``), "silu_glu", or "relu2" (no gate: w_gu [E, ff, W] holds the up rows alone);
+    ``in_w`` fp32 [T, top] (silu_glu only): choice k runs on
     in_w[t, k] h[t] (the experts have no biases, so the weight is applied to the gate and up
-    projections' outputs in fp32)."""
+    projections' outputs in fp32).  ``sorted_rows``: returns (outputs, rows) where rows int32 [T, top] names each
+    choice's row of the outputs viewed [-1, W] (prompt-sized steps leave them sorted by expert), or None when
+    they are in [T, top] order already."""
     T, top = idx.shape
     E, ff2, W = w_gu.shape
-    assert act in ("glu_clamp", "silu_glu") and (in_w is None or act == "silu_glu")
+    assert act in ("glu_clamp", "silu_glu", "relu2") and (in_w is None or act == "silu_glu")
     if _gpu(h):
         if T >= MOE_GEMM_MIN:
-            return _moe_experts_sorted(h, idx, w_gu, w_down, limit, act, in_w)
-        return _ext().sm_moe_experts(h, idx, w_gu, w_down, float(limit), act == "silu_glu", in_w)
+            return _moe_experts_sorted(h, idx, w_gu, w_down, limit, act, in_w, sorted_rows)
+        out = _ext().sm_moe_experts_relu2(h, idx, w_gu, w_down, None, None)[0] if act == "relu2" else \
+            _ext().sm_moe_experts(h, idx, w_gu, w_down, float(limit), act == "silu_glu", in_w)
+        return (out, None) if sorted_rows else out
     out = torch.zeros(T, top, w_down.shape[1], dtype=h.dtype, device=h.device)
     for e in idx.unique().tolist():
         t, k = (idx == e).nonzero(as_tuple=True)
         u = F.linear(h[t], w_gu[e])
-        y = glu_clamp(u, ff2 // 2, limit) if act == "glu_clamp" else \
+        y = relu2(u) if act == "relu2" else glu_clamp(u, ff2 // 2, limit) if act == "glu_clamp" else \
             glu_silu(u, ff2 // 2, None if in_w is None else in_w[t, k])
         out[t, k] = F.linear(y, w_down[e])
-    return out
+    return (out, None) if sorted_rows else out
 
 
-def _moe_experts_sorted(h, idx, w_gu, w_down, limit, act="glu_clamp", in_w=None):
+def moe_experts_shared(h: torch.Tensor, idx: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, shared_up: torch.Tensor,
+                       shared_down: torch.Tensor):
+    """Squared-ReLU experts and the shared expert of the same form in one go, for decode-sized steps: w_up
+    [E, ff, W], w_down [E, W, ff], shared_up [sff, W], shared_down [W, sff] -> (the chosen experts' outputs
+    [T, top, W], the shared expert's [T, W])."""
+    if _gpu(h):
+        return _ext().sm_moe_experts_relu2(h, idx, w_up, w_down, shared_up, shared_down)
+    return moe_experts(h, idx, w_up, w_down, 0.0, "relu2"), F.linear(relu2(F.linear(h, shared_up)), shared_down)
+
+
+def _moe_experts_sorted(h, idx, w_gu, w_down, limit, act="glu_clamp", in_w=None, sorted_rows=False):
     """Prompt-sized steps: (token, choice) pairs sorted by expert; every expert's rows run through its
     gate | up weights, one activation launch covers all rows, every expert's rows run through its down
     weights, and the rows go back to (token, choice) order.  bf16 on the GPU: the library's grouped
@@ -730,8 +841,9 @@ def _moe_experts_sorted(h, idx, w_gu, w_down, limit, act="glu_clamp", in_w=None)
     counts = torch.bincount(flat, minlength=E)
     rows = h.index_select(0, order // top)
     row_w = in_w.reshape(-1).index_select(0, order) if in_w is not None else None
-    glu = (lambda u_: glu_clamp(u_, ff2 // 2, limit)) if act == "glu_clamp" else (lambda u_: glu_silu(u_, ff2 // 2, row_w))
-    if h.is_cuda and h.dtype == torch.bfloat16 and W % 8 == 0 and ff2 % 16 == 0 and hasattr(torch, "_grouped_mm"):
+    glu = relu2 if act == "relu2" else (lambda u_: glu_clamp(u_, ff2 // 2, limit)) if act == "glu_clamp" else \
+        (lambda u_: glu_silu(u_, ff2 // 2, row_w))
+    if h.is_cuda and h.dtype == torch.bfloat16 and W % 8 == 0 and w_down.shape[2] % 8 == 0 and hasattr(torch, "_grouped_mm"):
         ends = torch.cumsum(counts, 0).to(torch.int32)
         y = glu(torch._grouped_mm(rows, w_gu.transpose(1, 2), offs=ends))
         o = torch._grouped_mm(y, w_down.transpose(1, 2), offs=ends)
@@ -747,9 +859,60 @@ def _moe_experts_sorted(h, idx, w_gu, w_down, limit, act="glu_clamp", in_w=None)
         y = glu(u)
         for e, a, n in spans:
             torch.mm(y[a:a + n], w_down[e].t(), out=o[a:a + n])
+    if sorted_rows:
+        back = torch.empty(T * top, dtype=torch.int32, device=h.device)
+        back[order] = torch.arange(T * top, dtype=torch.int32, device=h.device)
+        return o.view(T, top, -1), back.view(T, top)
     back = torch.empty_like(order)
     back[order] = torch.arange(T * top, device=h.device)
     return o.index_select(0, back).view(T, top, -1)
+
+
+# --------------------------------------------------------------------------- mixer and feed-forward side by side
+def embedding_learned(ids: torch.Tensor, meta: RaggedMeta, table: torch.Tensor, pos_table: torch.Tensor) -> torch.Tensor:
+    """fp32 rows ``table[id] + pos_table[position]``."""
+    if _gpu(table):
+        return _ext().sm_embed_learned(ids.long().contiguous(), table, pos_table, meta.tok_pos)
+    return table[ids.long()].float() + pos_table[meta.tok_pos.long()].float()
+
+
+def dynamic_tanh(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, alpha: torch.Tensor, out_dtype) -> torch.Tensor:
+    """tanh(alpha x) weight + bias in fp32 (PyTorch form; the GPU computes it inside ``parallel_update``)."""
+    return (torch.tanh(x * alpha.float()) * weight.float() + bias.float()).to(out_dtype)
+
+
+def parallel_update(x: torch.Tensor, norms: tuple, out_dtype, m: Optional[torch.Tensor] = None,
+                    m_scale: Optional[torch.Tensor] = None, y: Optional[torch.Tensor] = None, y_w: Optional[torch.Tensor] = None,
+                    parts: Optional[torch.Tensor] = None, part_w: Optional[torch.Tensor] = None,
+                    part_rows: Optional[torch.Tensor] = None, f_scale: Optional[torch.Tensor] = None) -> tuple:
+    """x (fp32 [T, W], in place) += m_scale m + f_scale (y_w y + sum_k part_w[:, k] parts_k), summed in fp32 in
+    this order, and the Dynamic Tanh norms ``norms`` = ((weight, bias, alpha), ..) (up to two) of the new x, each
+    as ``out_dtype`` [T, W]: what the next layer's mixer and feed-forward read, in the same pass.
+
+    ``m`` [T, W] the mixer's output; ``y`` [T, W] with ``y_w`` fp32 [T] (None: 1) a dense unit's or a shared
+    expert's; ``parts`` [T, K, W] with ``part_w`` fp32 [T, K] the chosen experts', choice k of token t at row
+    ``part_rows[t, k]`` of parts viewed [-1, W] (None: t K + k).  The scales are fp32 [W] (None: 1).  Without
+    m, y and parts x stays as it is and only the norms are computed."""
+    if _gpu(x):
+        return tuple(_ext().sm_parallel_update(x, m, m_scale, y, y_w, parts, part_w, part_rows, f_scale,
+                                               [t for n in norms for t in n], out_dtype == torch.float32))
+    if m is not None:
+        x.add_(m.float() if m_scale is None else m.float() * m_scale.float())
+    if y is not None or parts is not None:
+        v = torch.zeros_like(x) if y is None else y.float() if y_w is None else y_w[:, None] * y.float()
+        if parts is not None:
+            p = parts if part_rows is None else parts.reshape(-1, x.shape[1])[part_rows.long()]
+            for k in range(p.shape[1]):
+                v = v + part_w[:, k:k + 1] * p[:, k].float()
+        x.add_(v if f_scale is None else v * f_scale.float())
+    return tuple(dynamic_tanh(x, *n, out_dtype) for n in norms)
+
+
+def glu_gelu(u: torch.Tensor, ff: int) -> torch.Tensor:
+    """u [T, gate | up] -> gelu(gate) up with the tanh form of gelu (fp32 math, stored in u's dtype)."""
+    if _gpu(u):
+        return _ext().sm_glu_gelu(u, int(ff))
+    return (F.gelu(u[:, :ff].float(), approximate="tanh") * u[:, ff:2 * ff].float()).to(u.dtype)
 
 
 # --------------------------------------------------------------------------- residual streams
