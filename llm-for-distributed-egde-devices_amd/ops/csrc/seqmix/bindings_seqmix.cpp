@@ -97,6 +97,35 @@ int edge_sm_unrotate_gate(const void* a, const void* gate, int gate_ld, const in
 int edge_sm_moe_experts(const void* h, int W, const int* idx, int top, const void* w_gu, const void* w_down, int ff,
                         float limit, int silu, const float* in_w, void* y, void* out, int rows, int E, int f32,
                         hipStream_t st);
+int edge_sm_embed_learned(const int64_t* ids, const void* table, const void* pos_table, const int* tok_pos, float* out, int rows,
+                          int W, int V, int positions, int f32, hipStream_t st);
+int edge_sm_parallel_update(float* x, const void* m, const float* m_scale, const void* y, const float* y_w, const void* parts,
+                            const float* part_w, const int* part_rows, int K, int part_total, const float* f_scale,
+                            const float* const* norms, void* const* h, int nn, int rows, int W, int f32, hipStream_t st);
+int edge_sm_glu_gelu(const void* u, int ld, void* y, int rows, int ff, int f32, hipStream_t st);
+int edge_sm_moe_route_grouped(const void* h, int W, const float* router, int E, int gate, const float* corr, int groups,
+                              int keep, int top, float scale, float* z, int* idx, float* wts, float* gate_w, int rows, int f32,
+                              hipStream_t st);
+int edge_sm_moe_experts_relu2(const void* h, int W, const int* idx, int top, const void* w_up, const void* w_down, int ff,
+                              const void* su, const void* sd, int sff, void* y, void* ys, void* out, void* out_sh, int rows,
+                              int E, int f32, hipStream_t st);
+int edge_sm_latent_expand_write(const void* u, int ld, int c0, const float* w, float eps, const void* q, const void* uk,
+                                const int* tok_seq, const int* tok_pos, const int* seq_slot, const int* ptab, int ptab_ld,
+                                const float* cs, void* pages, void* qc, int rows, int H, int D, int R, int kvr, int rot, int page,
+                                int f32, hipStream_t st);
+int edge_sm_head_expand_gate(const void* a, const void* uv, const void* gate, int gate_ld, void* out, int rows, int H, int R,
+                             int Dv, int f32, hipStream_t st);
+int edge_sm_heads_gate(const void* v, const void* gate, int gate_ld, void* out, int rows, int H, int Dv, int f32,
+                       hipStream_t st);
+int edge_sm_gla_fused(int P);
+int edge_sm_gla_step_ok(int N);
+int edge_sm_gla_step(const void* u, int ld, const float* a2, const float* b, int rank, const float* norm_w, float* state,
+                     const int* seq_slot, const int* seq_start, const int* seq_len, const int* seq_off, void* out, float* y,
+                     int rows, int n, int H, int N, int P, float inv_tau, float eps, int f32, hipStream_t st);
+int edge_sm_gla_chunked(const void* u, int ld, const float* a2, const float* b, int rank, const float* norm_w, float* state,
+                        const int* seq_slot, const int* seq_start, const int* seq_len, const int* seq_off, void* out,
+                        float* la, float* sloc, float* cdec, float* y, int rows, int n, int max_chunks, int H, int N, int P,
+                        float inv_tau, float eps, int f32, hipStream_t st);
 }
 
 namespace {
@@ -901,6 +930,250 @@ at::Tensor sm_unrotate_gate(const at::Tensor& a, const std::optional<at::Tensor>
   return out;
 }
 
+// ---------------------------------------------------------------------------------- mixer and feed-forward side by side
+at::Tensor sm_embed_learned(const at::Tensor& ids, const at::Tensor& table, const at::Tensor& pos_table,
+                            const at::Tensor& tok_pos) {
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.dim() == 1, "ids: int64 [T]");
+  chk_act2(table, "table");
+  chk_act2(pos_table, "pos_table");
+  chk_i32(tok_pos, "tok_pos");
+  TORCH_CHECK(pos_table.scalar_type() == table.scalar_type() && pos_table.size(1) == table.size(1) &&
+                  tok_pos.numel() == ids.size(0), "pos_table [positions, W] like table, tok_pos [T]");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(table.device());
+  auto out = at::empty({ids.size(0), table.size(1)}, table.options().dtype(at::kFloat));
+  check(edge_sm_embed_learned(ids.data_ptr<int64_t>(), table.data_ptr(), pos_table.data_ptr(), tok_pos.data_ptr<int>(),
+                              out.data_ptr<float>(), (int)ids.size(0), (int)table.size(1), (int)table.size(0),
+                              (int)pos_table.size(0), f32(table), stream()), "sm_embed_learned");
+  return out;
+}
+
+// norms: (weight, bias, alpha) of up to two Dynamic Tanh norms, flat
+std::vector<at::Tensor> sm_parallel_update(at::Tensor& x, const std::optional<at::Tensor>& m,
+                                           const std::optional<at::Tensor>& m_scale, const std::optional<at::Tensor>& y,
+                                           const std::optional<at::Tensor>& y_w, const std::optional<at::Tensor>& parts,
+                                           const std::optional<at::Tensor>& part_w, const std::optional<at::Tensor>& part_rows,
+                                           const std::optional<at::Tensor>& f_scale, const std::vector<at::Tensor>& norms,
+                                           bool out_f32) {
+  chk_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2 && norms.size() % 3 == 0 && norms.size() <= 6, "x fp32 [T, W], up to two (weight, bias, alpha)");
+  const int64_t T = x.size(0), W = x.size(1);
+  auto act = [&](const std::optional<at::Tensor>& t, const char* name) -> const void* {
+    if (!t) return nullptr;
+    chk_act2(*t, name);
+    TORCH_CHECK(t->size(0) == T && t->size(1) == W && f32(*t) == (int)out_f32, name, ": [T, W] in the activation dtype");
+    return t->data_ptr();
+  };
+  auto vec = [&](const std::optional<at::Tensor>& t, int64_t n, const char* name) -> const float* {
+    if (!t) return nullptr;
+    chk_f32(*t, name);
+    TORCH_CHECK(t->numel() == n, name, ": wrong size");
+    return t->data_ptr<float>();
+  };
+  int64_t K = 0, total = 0;
+  if (parts) {
+    TORCH_CHECK(parts->is_cuda() && parts->is_contiguous() && parts->dim() == 3 && parts->size(0) == T && parts->size(2) == W &&
+                    is_act(*parts) && f32(*parts) == (int)out_f32 && part_w, "parts: [T, K, W] in the activation dtype, with weights");
+    K = parts->size(1);
+    total = T * K;
+    if (part_rows) {
+      chk_i32(*part_rows, "part_rows");
+      TORCH_CHECK(part_rows->numel() == total, "part_rows: int32 [T, K]");
+    }
+  }
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(x.device());
+  std::vector<at::Tensor> h;
+  const float* np[6];
+  void* hp[2] = {nullptr, nullptr};
+  const int nn = (int)(norms.size() / 3);
+  for (int i = 0; i < nn; ++i) {
+    for (int j = 0; j < 3; ++j) {
+      const at::Tensor& t = norms[3 * i + j];
+      chk_f32(t, "norm");
+      TORCH_CHECK(t.numel() == (j == 2 ? 1 : W), "norm: weight [W], bias [W], alpha [1]");
+      np[3 * i + j] = t.data_ptr<float>();
+    }
+    h.push_back(at::empty({T, W}, x.options().dtype(act_type(out_f32))));
+    hp[i] = h.back().data_ptr();
+  }
+  check(edge_sm_parallel_update(x.data_ptr<float>(), act(m, "m"), vec(m_scale, W, "m_scale"), act(y, "y"), vec(y_w, T, "y_w"),
+                                parts ? parts->data_ptr() : nullptr, parts ? vec(part_w, T * K, "part_w") : nullptr,
+                                parts && part_rows ? part_rows->data_ptr<int>() : nullptr, (int)K, (int)total,
+                                vec(f_scale, W, "f_scale"), np, hp, nn, (int)T, (int)W, out_f32, stream()),
+        "sm_parallel_update");
+  return h;
+}
+
+at::Tensor sm_glu_gelu(const at::Tensor& u, int64_t ff) {
+  TORCH_CHECK(is_act(u), "u: fp32 / bf16");
+  const int ld = row_ld(u, "u");
+  TORCH_CHECK(ff >= 0 && 2 * ff <= u.size(1), "u: [T, gate | up]");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(u.device());
+  auto y = at::empty({u.size(0), ff}, u.options());
+  check(edge_sm_glu_gelu(u.data_ptr(), ld, y.data_ptr(), (int)u.size(0), (int)ff, f32(u), stream()), "sm_glu_gelu");
+  return y;
+}
+
+std::tuple<at::Tensor, at::Tensor, at::Tensor> sm_moe_route_grouped(const at::Tensor& h, const at::Tensor& router,
+                                                                    const std::optional<at::Tensor>& corr, int64_t top,
+                                                                    double scale, int64_t groups, int64_t keep, bool gate) {
+  chk_act2(h, "h");
+  chk_f32(router, "router");
+  TORCH_CHECK(router.dim() == 2 && router.size(1) == h.size(1) && router.size(0) > (gate ? 1 : 0), "router: fp32 [E (+ 1), W]");
+  const int64_t T = h.size(0), E = router.size(0) - (gate ? 1 : 0);
+  if (corr) {
+    chk_f32(*corr, "correction");
+    TORCH_CHECK(corr->numel() == E, "correction: fp32 [E]");
+  }
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(h.device());
+  auto idx = at::empty({T, top}, h.options().dtype(at::kInt));
+  auto wts = at::empty({T, top}, h.options().dtype(at::kFloat));
+  auto gw = at::empty({gate ? T : 0}, wts.options());
+  auto z = at::empty({T, router.size(0)}, wts.options());
+  check(edge_sm_moe_route_grouped(h.data_ptr(), (int)h.size(1), router.data_ptr<float>(), (int)E, gate ? 1 : 0,
+                                  corr ? corr->data_ptr<float>() : nullptr, (int)groups, (int)keep, (int)top, (float)scale,
+                                  z.data_ptr<float>(), idx.data_ptr<int>(), wts.data_ptr<float>(),
+                                  gate ? gw.data_ptr<float>() : nullptr, (int)T, f32(h), stream()), "sm_moe_route_grouped");
+  return {idx, wts, gw};
+}
+
+std::tuple<at::Tensor, at::Tensor> sm_moe_experts_relu2(const at::Tensor& h, const at::Tensor& idx, const at::Tensor& w_up,
+                                                        const at::Tensor& w_down, const std::optional<at::Tensor>& su,
+                                                        const std::optional<at::Tensor>& sd) {
+  chk_act2(h, "h");
+  chk_i32(idx, "idx");
+  const int64_t T = h.size(0), W = h.size(1);
+  TORCH_CHECK(idx.dim() == 2 && idx.size(0) == T, "idx: int32 [T, top]");
+  TORCH_CHECK(w_up.is_cuda() && w_up.is_contiguous() && w_up.dim() == 3 && w_up.size(2) == W && w_down.is_cuda() &&
+                  w_down.is_contiguous() && w_down.dim() == 3 && w_down.size(0) == w_up.size(0) && w_down.size(1) == W &&
+                  w_down.size(2) == w_up.size(1) && w_up.scalar_type() == h.scalar_type() &&
+                  w_down.scalar_type() == h.scalar_type(), "experts: w_up [E, ff, W], w_down [E, W, ff]");
+  int64_t sff = 0;
+  TORCH_CHECK(bool(su) == bool(sd), "the shared expert has two matrices");
+  if (su) {
+    chk_act2(*su, "shared up");
+    chk_act2(*sd, "shared down");
+    sff = su->size(0);
+    TORCH_CHECK(su->size(1) == W && sd->size(0) == W && sd->size(1) == sff && su->scalar_type() == h.scalar_type() &&
+                    sd->scalar_type() == h.scalar_type(), "shared expert: up [sff, W], down [W, sff]");
+  }
+  const int64_t top = idx.size(1), ff = w_up.size(1);
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(h.device());
+  auto y = at::empty({T * top, ff}, h.options());
+  auto ys = at::empty({sff ? T : 0, sff}, h.options());
+  auto out = at::empty({T, top, W}, h.options());
+  auto out_sh = at::empty({sff ? T : 0, W}, h.options());
+  check(edge_sm_moe_experts_relu2(h.data_ptr(), (int)W, idx.data_ptr<int>(), (int)top, w_up.data_ptr(), w_down.data_ptr(),
+                                  (int)ff, su ? su->data_ptr() : nullptr, sd ? sd->data_ptr() : nullptr, (int)sff, y.data_ptr(),
+                                  sff ? ys.data_ptr() : nullptr, out.data_ptr(), sff ? out_sh.data_ptr() : nullptr, (int)T,
+                                  (int)w_up.size(0), f32(h), stream()), "sm_moe_experts_relu2");
+  return {out, out_sh};
+}
+
+at::Tensor sm_latent_expand_write(const at::Tensor& u, int64_t c0, const at::Tensor& w, double eps, const at::Tensor& q,
+                                  const at::Tensor& uk, const at::Tensor& tok_seq, const at::Tensor& tok_pos,
+                                  const at::Tensor& seq_slot, const at::Tensor& ptab, const std::optional<at::Tensor>& cs,
+                                  at::Tensor& pages, int64_t rot) {
+  chk_i32(tok_seq, "tok_seq");
+  chk_i32(tok_pos, "tok_pos");
+  chk_i32(seq_slot, "seq_slot");
+  chk_table(ptab);
+  chk_f32(w, "latent norm weight");
+  const int ld = row_ld(u, "u");
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && is_act(q), "q: [T, H, D + R]");
+  TORCH_CHECK(uk.is_cuda() && uk.dim() == 3 && uk.is_contiguous() && uk.scalar_type() == q.scalar_type() &&
+                  uk.size(0) == q.size(1) && uk.size(1) <= q.size(2), "uk: [H, D, kv_rank]");
+  const int64_t T = q.size(0), H = q.size(1), D = uk.size(1), R = q.size(2) - D, kvr = uk.size(2), page = pages.size(1);
+  TORCH_CHECK(pages.is_cuda() && pages.is_contiguous() && pages.dim() == 4 && pages.size(2) == 1 &&
+                  pages.scalar_type() == q.scalar_type() && pages.size(3) == kvr + R, "pages: [pages, page, 1, kv_rank + R]");
+  TORCH_CHECK(u.scalar_type() == q.scalar_type() && u.size(0) == T && c0 >= 0 && c0 + kvr + R <= u.size(1) && w.numel() == kvr,
+              "u: [T, .. latent | key part ..]");
+  TORCH_CHECK(tok_seq.numel() == T && tok_pos.numel() == T, "metadata sizes");
+  if (rot > 0) {
+    TORCH_CHECK(cs, "rotary table missing");
+    chk_f32(*cs, "rotary table");
+    TORCH_CHECK(cs->dim() == 3 && cs->size(1) == rot / 2 && cs->size(2) == 2, "rotary table: [positions, rot / 2, 2]");
+  }
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(q.device());
+  auto qc = at::empty({T, H, kvr + R}, q.options());
+  check(edge_sm_latent_expand_write(u.data_ptr(), ld, (int)c0, w.data_ptr<float>(), (float)eps, q.data_ptr(), uk.data_ptr(),
+                                    tok_seq.data_ptr<int>(), tok_pos.data_ptr<int>(), seq_slot.data_ptr<int>(),
+                                    ptab.data_ptr<int>(), (int)ptab.stride(0), rot > 0 ? cs->data_ptr<float>() : nullptr,
+                                    pages.data_ptr(), qc.data_ptr(), (int)T, (int)H, (int)D, (int)R, (int)kvr, (int)rot,
+                                    (int)page, f32(q), stream()), "sm_latent_expand_write");
+  return qc;
+}
+
+at::Tensor sm_head_expand_gate(const at::Tensor& a, const at::Tensor& uv, const std::optional<at::Tensor>& gate) {
+  chk_act2(a, "a");
+  TORCH_CHECK(uv.is_cuda() && uv.dim() == 3 && uv.is_contiguous() && uv.scalar_type() == a.scalar_type() &&
+                  a.size(1) == uv.size(0) * uv.size(1), "a [T, H R], uv [H, R, Dv]");
+  const int64_t T = a.size(0), H = uv.size(0), R = uv.size(1), Dv = uv.size(2);
+  int gate_ld = 0;
+  if (gate) {
+    gate_ld = row_ld(*gate, "gate");
+    TORCH_CHECK(gate->size(0) == T && gate->size(1) == H * Dv && gate->scalar_type() == a.scalar_type(), "gate: [T, H Dv]");
+  }
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(a.device());
+  auto out = at::empty({T, H * Dv}, a.options());
+  check(edge_sm_head_expand_gate(a.data_ptr(), uv.data_ptr(), gate ? gate->data_ptr() : nullptr, gate_ld, out.data_ptr(), (int)T,
+                                 (int)H, (int)R, (int)Dv, f32(a), stream()), "sm_head_expand_gate");
+  return out;
+}
+
+at::Tensor sm_heads_gate(const at::Tensor& v, const at::Tensor& gate) {
+  TORCH_CHECK(v.is_cuda() && v.dim() == 3 && v.is_contiguous() && is_act(v), "v: [H, T, Dv]");
+  const int gate_ld = row_ld(gate, "gate");
+  const int64_t H = v.size(0), T = v.size(1), Dv = v.size(2);
+  TORCH_CHECK(gate.size(0) == T && gate.size(1) == H * Dv && gate.scalar_type() == v.scalar_type(), "gate: [T, H Dv]");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(v.device());
+  auto out = at::empty({T, H * Dv}, v.options());
+  check(edge_sm_heads_gate(v.data_ptr(), gate.data_ptr(), gate_ld, out.data_ptr(), (int)T, (int)H, (int)Dv, f32(v), stream()),
+        "sm_heads_gate");
+  return out;
+}
+
+// chunks > 0: the form over 64-token chunks (chunks = sum of ceil(len / 64), max_chunks = the largest of them)
+at::Tensor sm_gla(const at::Tensor& u, const at::Tensor& a2, const at::Tensor& b, const at::Tensor& norm_w, at::Tensor& state,
+                  const at::Tensor& seq_slot, const at::Tensor& seq_start, const at::Tensor& seq_len, const at::Tensor& seq_off,
+                  int64_t n, int64_t H, int64_t N, int64_t P, double tau, double eps, int64_t chunks, int64_t max_chunks) {
+  TORCH_CHECK(is_act(u), "u: fp32 / bf16");
+  const int ld = row_ld(u, "u");
+  chk_f32(a2, "a2");
+  chk_f32(b, "decay bias");
+  chk_f32(norm_w, "norm weight");
+  chk_f32(state, "state");
+  for (const at::Tensor* t : {&seq_slot, &seq_start, &seq_len, &seq_off}) chk_i32(*t, "metadata");
+  const int64_t T = u.size(0), rank = a2.size(1);
+  TORCH_CHECK(a2.dim() == 2 && a2.size(0) == H * N && b.numel() == H * N && norm_w.numel() == P && rank >= 1 &&
+                  u.size(1) == 2 * H * N + 2 * H * P + rank && tau > 0, "u [T, q | k | v | gate | decay down], a2 [H N, rank]");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == N && state.size(3) == P,
+              "state: fp32 [slots, heads, N, P]");
+  TORCH_CHECK(seq_slot.numel() >= n && seq_start.numel() >= n && seq_len.numel() >= n && seq_off.numel() >= n,
+              "sequence metadata: [n]");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(u.device());
+  auto out = at::empty({T, H * P}, u.options());
+  auto f = u.options().dtype(at::kFloat);
+  at::Tensor y;
+  if (!edge_sm_gla_fused((int)P)) y = at::empty({T, H * P}, f);
+  float* yp = y.defined() ? y.data_ptr<float>() : nullptr;
+  TORCH_CHECK(chunks > 0 || edge_sm_gla_step_ok((int)N), "key channels per head: the token-by-token form takes up to 256");
+  if (chunks > 0) {
+    TORCH_CHECK(chunks * 64 >= T && max_chunks > 0 && max_chunks <= chunks, "chunk counts do not cover the step");
+    auto la = at::empty({T, H * N}, f), sloc = at::empty({chunks, H, N, P}, f), cdec = at::empty({chunks, H, N}, f);
+    check(edge_sm_gla_chunked(u.data_ptr(), ld, a2.data_ptr<float>(), b.data_ptr<float>(), (int)rank, norm_w.data_ptr<float>(),
+                              state.data_ptr<float>(), seq_slot.data_ptr<int>(), seq_start.data_ptr<int>(),
+                              seq_len.data_ptr<int>(), seq_off.data_ptr<int>(), out.data_ptr(), la.data_ptr<float>(),
+                              sloc.data_ptr<float>(), cdec.data_ptr<float>(), yp, (int)T, (int)n, (int)max_chunks, (int)H, (int)N,
+                              (int)P, (float)(1.0 / tau), (float)eps, f32(u), stream()), "sm_gla_chunked");
+    return out;
+  }
+  check(edge_sm_gla_step(u.data_ptr(), ld, a2.data_ptr<float>(), b.data_ptr<float>(), (int)rank, norm_w.data_ptr<float>(),
+                         state.data_ptr<float>(), seq_slot.data_ptr<int>(), seq_start.data_ptr<int>(), seq_len.data_ptr<int>(),
+                         seq_off.data_ptr<int>(), out.data_ptr(), yp, (int)T, (int)n, (int)H, (int)N, (int)P,
+                         (float)(1.0 / tau), (float)eps, f32(u), stream()), "sm_gla_step");
+  return out;
+}
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -936,4 +1209,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("sm_poly_norm", &sm_poly_norm);
   m.def("sm_qk_norm_rope_write", &sm_qk_norm_rope_write);
   m.def("sm_unrotate_gate", &sm_unrotate_gate);
+  m.def("sm_embed_learned", &sm_embed_learned);
+  m.def("sm_parallel_update", &sm_parallel_update);
+  m.def("sm_glu_gelu", &sm_glu_gelu);
+  m.def("sm_moe_route_grouped", &sm_moe_route_grouped);
+  m.def("sm_moe_experts_relu2", &sm_moe_experts_relu2);
+  m.def("sm_latent_expand_write", &sm_latent_expand_write);
+  m.def("sm_head_expand_gate", &sm_head_expand_gate);
+  m.def("sm_heads_gate", &sm_heads_gate);
+  m.def("sm_gla", &sm_gla);
 }

@@ -633,7 +633,7 @@ def gated_linear_attention(u: torch.Tensor, a2: torch.Tensor, a2_b: torch.Tensor
         # portions of GLA_CHUNK_MIN tokens or more: kernels parallel over 64-token chunks; shorter steps (decode):
         # one workgroup per (sequence, head), token by token, with the decays, the norm and the gate in it
         chunks = max_chunks = 0
-        if meta.max_len >= GLA_CHUNK_MIN:
+        if meta.max_len >= GLA_CHUNK_MIN or N > 256:
             per = [(h[2] + 63) // 64 for h in meta.host]
             chunks, max_chunks = sum(per), max(per)
         return _ext().sm_gla(u, a2, a2_b, norm_w, state, meta.seq_slot, meta.seq_start, meta.seq_len, meta.seq_off,
