@@ -349,6 +349,8 @@ class HybridLM(nn.Module):
         one ragged prompt pass through a cache of its own."""
         from .. import ops
         from ..engine.ragged import RaggedEngine
+        if self.cfg.pos_emb == "learned":                # a text longer than the position table: its end
+            ids = ids[-self.cfg.max_position_embeddings:]
         eng = RaggedEngine(self, len(ids), slots=1, use_graphs=False)
         logits = eng.step([("c", list(ids), list(range(len(ids))))])
         return float(ops.max_softmax_prob(logits).mean())

@@ -648,8 +648,8 @@ def gated_linear_attention(u: torch.Tensor, a2: torch.Tensor, a2_b: torch.Tensor
         v = x[:, 2 * HN:2 * HN + HP].view(n, heads, P)
         S = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
         for t in range(n):
-            S = a[off + t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
-            y[off + t] = torch.einsum("hnp,hn->hp", S, q[t]).reshape(HP)
+            S.mul_(a[off + t][:, :, None]).add_(k[t][:, :, None] * v[t][:, None, :])
+            y[off + t] = torch.bmm(q[t][:, None, :], S).reshape(HP)
         state[slot] = S
     return head_norm_gate(y, u[:, 2 * HN + HP:2 * HN + 2 * HP], norm_w, heads, eps, u.dtype, act="silu")
 
