@@ -9,7 +9,10 @@ beside the Pagonex model of equal width, heads, state size and active expert wid
 (``--hybrid-family fikupel``) the Fikupel model (latent attention without positions and gated
 grouped-query attention with rotated values, both with a window and a sink, PolyNorm and expert
 feed-forwards, two residual streams) beside the Vetevik model of equal width, heads, head size, window
-and active expert width.
+and active expert width; or (``--hybrid-family numizen``) the Numizen model (gated latent attention and
+gated linear attention beside a gelu-gated unit or group-limited squared-ReLU experts) beside the Pagonex
+model of equal width, heads, head sizes, latent ranks, state size and active feed-forward work, its latent
+attention without a window as well.
 
 Sizes resemble real layers (random weights): the hybrid layer has windowed attention with pooled
 blocks + a Mamba-2 mixer + a squared-ReLU feed-forward; the comparison model is the
@@ -28,7 +31,7 @@ from typing import Dict, List
 
 import torch
 
-from ..models.configs import (ChunkAttnSpec, DeltaSpec, GatedAttnSpec, LatentAttnSpec, LayerSpec, ModelConfig, MoESpec,
+from ..models.configs import (ChunkAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, LatentAttnSpec, LayerSpec, ModelConfig, MoESpec,
                               SSDSpec, WindowAttnSpec, PRESETS)
 from ..models.decoder import build_model
 from ..models.hybrid import build_hybrid
@@ -150,6 +153,36 @@ def fikupel_config(s: dict) -> ModelConfig:
                        tie_word_embeddings=True, name="fikupel-bench", layer_specs=specs, streams=s["streams"], hyper=True)
 
 
+# Numizen sizes: latent-attention and linear-attention layers alternate with the heads, ranks and state sizes of the
+# Pagonex size of the same name; a squared-ReLU expert has two matrices where Pagonex's gated one has three, so
+# experts half as wide again make the active work equal; the first layer's dense unit is as wide as Pagonex's
+# three experts + shared one
+NUMIZEN_SIZES = {
+    "w1024": dict(width=1024, layers=4, heads=16, dim=64, rot=32, vdim=64, q_rank=384, kv_rank=128, l_heads=16, l_dim=64,
+                  l_vdim=64, rank=16, experts=16, top=3, groups=4, keep=2, ff=1536, shared=1536, dense_ff=4096, vocab=32000),
+    "w2048": dict(width=2048, layers=4, heads=16, dim=128, rot=64, vdim=128, q_rank=768, kv_rank=256, l_heads=16, l_dim=128,
+                  l_vdim=128, rank=16, experts=32, top=3, groups=4, keep=2, ff=3072, shared=3072, dense_ff=8192, vocab=32000),
+}
+
+
+def numizen_config(s: dict) -> ModelConfig:
+    moe = MoESpec(s["experts"], s["top"], 1.0, s["ff"], shared_ff=s["shared"], router="softmax", act="relu2", correction=True,
+                  groups=s["groups"], groups_keep=s["keep"], shared_gate=True)
+    specs = []
+    for i in range(s["layers"]):
+        ff = dict(ff=s["dense_ff"], ff_act="gelu_glu") if i == 0 else dict(moe=moe, ff_act="gelu_glu")
+        if i % 2 == 0:
+            a = LatentAttnSpec(s["heads"], s["dim"], s["rot"], s["vdim"], s["q_rank"], s["kv_rank"], (s["dim"] + s["rot"]) ** -0.5,
+                               None, s["rot"], 500000.0, gate=True)
+            specs.append(LayerSpec("latent_attention", latent=a, **ff))
+        else:
+            specs.append(LayerSpec("gla", gla=GLASpec(s["l_heads"], s["l_dim"], s["l_vdim"], 16.0, s["rank"]), **ff))
+    return ModelConfig(arch="numizen", vocab_size=s["vocab"], hidden_size=s["width"], num_layers=s["layers"],
+                       num_heads=s["heads"], num_kv_heads=1, intermediate_size=s["dense_ff"], head_dim=s["dim"],
+                       max_position_embeddings=1 << 15, norm="dyt", norm_eps=1e-6, act="gelu_tanh", parallel_residual=True,
+                       pos_emb="learned", name="numizen-bench", layer_specs=specs, layer_scale=True)
+
+
 def closest_config(s: dict) -> ModelConfig:
     return PRESETS["phi-2"].replace(vocab_size=s["vocab"], hidden_size=s["width"], num_layers=s["layers"],
                                     num_heads=s["heads"], num_kv_heads=s["kv"], head_dim=s["dim"], rotary_dim=s["dim"],
@@ -200,15 +233,25 @@ def op_times(eng: RaggedEngine, entries, close=()) -> Dict[str, float]:
              "embedding_bigram", "canon_conv", "layer_norm_rows", "layer_norm_residual", "rms_norm_cols", "glu_clamp",
              "latent_write", "delta_prepare", "delta_rule_scan", "head_norm_gate", "moe_route", "moe_experts",
              "group_rms_norm", "group_norm_residual", "chunk_attention", "delta_prepare_head", "glu_silu",
-             "hyper_read_norm", "hyper_update", "poly_norm", "qk_norm_rope_write", "unrotate_gate"]
+             "hyper_read_norm", "hyper_update", "poly_norm", "qk_norm_rope_write", "unrotate_gate",
+             "embedding_learned", "parallel_update", "glu_gelu", "moe_route_grouped", "moe_experts_shared",
+             "latent_expand_write", "head_expand_gate", "gated_linear_attention"]
     saved = {n: getattr(seqmix, n) for n in names}
     lin = F.linear
 
+    depth = [0]                                  # an op inside another op counts for the outer one
+
     def wrap(name, fn):
         def inner(*a, **k):
+            if depth[0]:
+                return fn(*a, **k)
+            depth[0] += 1
             e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
             e0.record()
-            r = fn(*a, **k)
+            try:
+                r = fn(*a, **k)
+            finally:
+                depth[0] -= 1
             e1.record()
             marks.append((name, e0, e1))
             return r
@@ -311,6 +354,23 @@ def run_fikupel(sizes: List[str], prompt: int, batch: int, steps: int, device) -
             "decode_batch": batch, "decode_steps": steps, "sizes": res}
 
 
+def run_numizen(sizes: List[str], prompt: int, batch: int, steps: int, device) -> Dict:
+    res = {}
+    r2 = lambda d: {k: (round(v, 2) if isinstance(v, float) else v) for k, v in d.items()}
+    for name in sizes:
+        s, c = NUMIZEN_SIZES[name], dict(PAGONEX_SIZES[name], window=None)
+        n = bench_hybrid(s, prompt, batch, steps, device, numizen_config(s))
+        torch.cuda.empty_cache()
+        p = bench_hybrid(c, prompt, batch, steps, device, pagonex_config(c))
+        torch.cuda.empty_cache()
+        res[name] = {"size": s, "closest_size": c, "numizen": r2(n), "closest_pagonex": r2(p),
+                     "prefill_ratio": round(n["prefill_tok_s"] / p["prefill_tok_s"], 3),
+                     "decode_ratio": round(n["decode_tok_s"] / p["decode_tok_s"], 3)}
+    return {"metric": "prefill / decode tokens/s, Numizen layer-spec model vs the Pagonex model of equal size",
+            "dtype": "bf16", "data": "synthetic (random weights, random prompt)", "prompt_tokens": prompt,
+            "decode_batch": batch, "decode_steps": steps, "sizes": res}
+
+
 def run(sizes: List[str], prompt: int = 4096, batch: int = 4, steps: int = 32, device=None, family: str = "nudadra") -> Dict:
     device = torch.device(device or "cuda:0")
     if family == "pagonex":
@@ -319,6 +379,8 @@ def run(sizes: List[str], prompt: int = 4096, batch: int = 4, steps: int = 32, d
         return run_vetevik(sizes, prompt, batch, steps, device)
     if family == "fikupel":
         return run_fikupel(sizes, prompt, batch, steps, device)
+    if family == "numizen":
+        return run_numizen(sizes, prompt, batch, steps, device)
     res = {}
     for name in sizes:
         s = SIZES[name]

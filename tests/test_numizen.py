@@ -393,7 +393,7 @@ GLA_CASES = [  # heads, dim, vdim, tau, rank, decay bias, lengths
     (2, 33, 70, 4.0, 3, 2.0, (131, 64)),
     (1, 100, 130, 16.0, 16, 3.0, (150, 30)),           # a head wider than one workgroup's columns
     (2, 200, 96, 2.0, 8, 4.0, (140, 24)),
-    (4, 16, 32, 0.25, 5, -4.0, (130, 17)),             # forgets within a token: the state underflows
+    (4, 16, 32, 0.25, 37, -4.0, (130, 17)),            # forgets within a token: the state underflows
     (2, 40, 24, 1.0, 2, -12.0, (129, 70)),             # a 16-token block decays by far more than fp32's range
     (1, 260, 16, 16.0, 4, 2.0, (70, 5)),               # more key channels than the token-by-token kernel holds
 ]
