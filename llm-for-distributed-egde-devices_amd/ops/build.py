@@ -26,8 +26,10 @@ BUILD = os.path.join(HERE, "..", "..", "build", "ops")
 ARCH = os.environ.get("EDGELLM_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 
+# hipcc -O3 forms packed fp32 instructions from plain float code; some of their forms have given wrong results on
+# this hardware, so no kernel is built with them
 KERNEL_FLAGS = ["-O3", "-fPIC", "-std=c++17", f"--offload-arch={ARCH}", "-munsafe-fp-atomics",
-                "-Wno-unused-result"]
+                "-Wno-unused-result", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _torch_paths():
@@ -39,11 +41,7 @@ def _torch_paths():
     return inc, lib, abi
 
 
-# hipcc -O3 forms packed fp32 instructions from plain float code; the ragged-step kernels are built
-# without them (their fp32 results are compared at 1e-5)
-SEQMIX_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
-
-TARGETS = {"main": ("_C", CSRC, []), "seqmix": ("_seqmix", os.path.join(CSRC, "seqmix"), SEQMIX_FLAGS)}
+TARGETS = {"main": ("_C", CSRC), "seqmix": ("_seqmix", os.path.join(CSRC, "seqmix"))}
 
 
 def target_path(target: str = "main") -> str:
@@ -73,7 +71,7 @@ def build(verbose: bool = False, jobs: int = 8, targets=("main", "seqmix")) -> s
 
 
 def _build_target(target: str, verbose: bool, jobs: int) -> str:
-    name, src_dir, extra = TARGETS[target]
+    name, src_dir = TARGETS[target]
     build_dir = BUILD if target == "main" else os.path.join(BUILD, target)
     os.makedirs(build_dir, exist_ok=True)
     inc, lib, abi = _torch_paths()
@@ -85,7 +83,7 @@ def _build_target(target: str, verbose: bool, jobs: int) -> str:
         src = os.path.join(src_dir, f)
         if f.endswith(".hip"):
             obj = os.path.join(build_dir, f[:-4] + ".o")
-            cmd = [HIPCC, *KERNEL_FLAGS, *extra, "-I", CSRC, "-c", src, "-o", obj]
+            cmd = [HIPCC, *KERNEL_FLAGS, "-I", CSRC, "-c", src, "-o", obj]
         elif f.endswith(".cpp"):
             obj = os.path.join(build_dir, f[:-4] + ".o")
             cmd = [HIPCC, "-O2", "-fPIC", "-std=c++17", "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1",

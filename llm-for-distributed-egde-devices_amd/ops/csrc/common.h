@@ -48,8 +48,12 @@ __device__ __forceinline__ float e2f(uint32_t u16) {
 }
 template <bool H>
 __device__ __forceinline__ uint16_t f2e(float f) {
-  if constexpr (H) return __half_as_ushort(__float2half(f));     // round to nearest even
-  else return f2bf(f);
+  if constexpr (H) {
+    // the fp32 value is rounded to fp16 as it stands: a multiply is not merged with its conversion (a mixed-precision
+    // FMA rounds once where other kernels round twice), so kernels that compute the same expression agree
+    asm("" : "+v"(f));
+    return __half_as_ushort(__float2half(f));                    // round to nearest even
+  } else return f2bf(f);
 }
 template <bool H>
 __device__ __forceinline__ uint32_t pack_e2(float lo, float hi) {

@@ -313,14 +313,19 @@ extern "C" int edge_llmint8_outlier(void* out, const float* xo, const int* cols,
   return (int)hipGetLastError();
 }
 
+// a kernel and not a memset node: callers may capture this into a graph
+__global__ void __launch_bounds__(256) llmint8_clear_kernel(uint32_t* flags, int words) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < words) flags[i] = 0u;
+}
+
 // Any-rows preparation: x bf16 [M, K] (K % 32 == 0) -> q int8 [M, K] (outlier columns zeroed),
 // sa [M], cols [K] (first *count), count [1]; flags / take: scratch of K / 32 words each.
 extern "C" int edge_llmint8_prep_rows(const void* x, int M, int K, float thr, void* q, float* sa, int* cols, int* count,
                                       uint32_t* flags, uint32_t* take, hipStream_t st) {
   if (M <= 0 || K % 32 != 0 || K <= 0) return -2;
   const int words = K / 32;
-  hipError_t e = hipMemsetAsync(flags, 0, (size_t)words * 4, st);
-  if (e != hipSuccess) return (int)e;
+  hipLaunchKernelGGL(llmint8_clear_kernel, dim3((words + 255) / 256), dim3(256), 0, st, flags, words);
   hipLaunchKernelGGL(llmint8_flags_kernel, dim3((K + 2047) / 2048, (M + FR_ROWS - 1) / FR_ROWS), dim3(256), 0, st,
                      (const bf16_t*)x, M, K, thr, flags);
   hipLaunchKernelGGL(llmint8_compact_kernel, dim3(1), dim3(64), 0, st, (const uint32_t*)flags, words, K, take, cols,
