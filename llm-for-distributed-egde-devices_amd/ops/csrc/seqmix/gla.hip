@@ -21,7 +21,6 @@
 
 namespace {
 
-constexpr int CL = 64;                                       // tokens per chunk
 constexpr float LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float log_sigmoid(float z) {
@@ -33,15 +32,6 @@ __device__ __forceinline__ float log2_sigmoid(float z) {
   return -(fmaxf(-z, 0.f) * LOG2E + __builtin_amdgcn_logf(1.f + ex2(-fabsf(z) * LOG2E)));
 }
 __device__ __forceinline__ v4f mfma4(float a, float b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-
-// sum over the 16 lanes of a DPP row; every lane gets it
-__device__ __forceinline__ float row16_sum(float v) {
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xF, 0xF, false));
-  return v;
-}
 
 // ---------------------------------------------------------------------------------- token by token
 // One workgroup of NW waves per (sequence, head, 64 CG value columns): lane = column, wave w keeps the state rows
@@ -137,12 +127,6 @@ __global__ void __launch_bounds__(64 * NW) gla_step_kernel(
 }
 
 // ---------------------------------------------------------------------------------- chunks
-__device__ __forceinline__ int chunk_base(const int* __restrict__ seq_len, int s) {
-  int b = 0;
-  for (int i = 0; i < s; ++i) b += (seq_len[i] + CL - 1) / CL;
-  return b;
-}
-
 // rows x cols of a tile to LDS rows of LDT floats, zeros past (rl, cl); VEC: 8 elements per access (cols, cl, the
 // source's stride and alignment allow it)
 // SWZ: the 16-column groups of row r are stored in the order g ^ (r mod 4), so four token rows of an operand hit

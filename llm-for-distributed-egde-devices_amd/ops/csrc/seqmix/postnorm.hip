@@ -4,7 +4,9 @@
 // column slice, the cached and the query side of latent attention (RMS norm, neighbour-pair rotation,
 // page-table scatter), the gated delta rule (unit-length q / k, decays, the token-by-token recurrence
 // over a [N, P] fp32 state per head, per-head norm with a sigmoid gate), the clamped gated-linear
-// activation, and the mixture of experts' router and decode-sized expert products.
+// activation, and the mixture of experts' routers and decode-sized expert products (gated-linear experts, or
+// squared-ReLU ones with the shared expert); also the two ends of latent attention on decode-sized steps: queries
+// through the key expansion + cache write, heads through the value expansion + gate.
 //
 // Storage is fp32 or bf16 (template T); norms, scores' inputs that the design keeps in 32-bit, decays,
 // the router and the recurrent state are fp32 in both.  A token is addressed by (sequence of the step,
@@ -241,6 +243,125 @@ __global__ void __launch_bounds__(NT) latent_write_kernel(const T* __restrict__ 
   }
 }
 
+// ---------------------------------------------------------------------------------- latent attention, few tokens
+// out_s[n] = sum_k x_s[k] M[k][n] (M row-major [K, N]) by the whole workgroup; red_s: 8 NT floats.  With N a
+// multiple of 8 a thread takes 8 columns of every (NT / (N / 8))-th row and the shares are added up in order.
+template <typename T>
+__device__ __forceinline__ void vec_mat(const float* x_s, const T* __restrict__ M, int K, int N, float* out_s, float* red_s) {
+  const int tid = threadIdx.x, cpr = N / 8;
+  if (N % 8 == 0 && cpr <= NT) {
+    const int ng = NT / cpr, g = tid / cpr, c = (tid % cpr) * 8;
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+    if (g < ng) {
+#pragma unroll 4
+      for (int k = g; k < K; k += ng) {
+        float m[8];
+        load8<T>(M + (size_t)k * N + c, m);
+        const float xv = x_s[k];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] += xv * m[e];
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) red_s[g * N + c + e] = acc[e];
+    }
+    __syncthreads();
+    for (int n = tid; n < N; n += NT) {
+      float s = 0.f;
+      for (int q = 0; q < ng; ++q) s += red_s[q * N + n];
+      out_s[n] = s;
+    }
+  } else {
+    for (int n = tid; n < N; n += NT) {
+      float s = 0.f;
+      for (int k = 0; k < K; ++k) s += x_s[k] * ldf<T>(M + (size_t)k * N + n);
+      out_s[n] = s;
+    }
+  }
+  __syncthreads();
+}
+
+// Workgroup (t, h < H): qc[t, h] = (sum_d q[t, h, d] uk[h, d, :]) | rotate(q[t, h, D : D + R]).  Workgroup (t, H): the
+// cached row rms(u[c0 : c0 + kvr]) w | rotate(u[c0 + kvr : ..]).  LDS: x [max(D, 1)] | out [kvr] | shares [8 NT].
+template <typename T>
+__global__ void __launch_bounds__(NT) latent_expand_write_kernel(
+    const T* __restrict__ u, int ld, int c0, const float* __restrict__ w, float eps, const T* __restrict__ q,
+    const T* __restrict__ uk, const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, const int* __restrict__ seq_slot,
+    const int* __restrict__ ptab, int ptab_ld, const float* __restrict__ cs, T* __restrict__ pages, T* __restrict__ qc, int H,
+    int D, int R, int kvr, int rot, int page) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  __shared__ float red[NT / 64];
+  const int t = blockIdx.x, h = blockIdx.y, pos = tok_pos[t], tid = threadIdx.x;
+  const float* c = cs ? cs + (size_t)pos * rot : nullptr;    // rot / 2 pairs of (cos, sin)
+  auto turned = [&](const T* v, int d) {                     // coordinate d of the rotated R-vector v
+    const float a = ldf<T>(v + d);
+    if (d >= rot || !c) return a;
+    const float o = ldf<T>(v + (d ^ 1)), co = c[d & ~1], si = c[(d & ~1) + 1];
+    return (d & 1) ? a * co + o * si : a * co - o * si;
+  };
+  if (h == H) {
+    const T* ur = u + (size_t)t * ld + c0;
+    float ss = 0.f;
+    for (int e = tid; e < kvr; e += NT) { const float v = ldf<T>(ur + e); ss += v * v; }
+    const float r = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)kvr + eps);
+    const int slot = seq_slot[tok_seq[t]];
+    T* row = pages + ((size_t)ptab[(size_t)slot * ptab_ld + pos / page] * page + pos % page) * (kvr + R);
+    for (int e = tid; e < kvr; e += NT) stf<T>(row + e, ldf<T>(ur + e) * r * w[e]);
+    for (int e = tid; e < R; e += NT) stf<T>(row + kvr + e, turned(ur + kvr, e));
+    return;
+  }
+  float *x_s = smem, *out_s = smem + D, *red_s = smem + D + kvr;
+  const T* qr = q + ((size_t)t * H + h) * (D + R);
+  T* dst = qc + ((size_t)t * H + h) * (kvr + R);
+  for (int d = tid; d < D; d += NT) x_s[d] = ldf<T>(qr + d);
+  __syncthreads();
+  vec_mat<T>(x_s, uk + (size_t)h * D * kvr, D, kvr, out_s, red_s);
+  for (int e = tid; e < kvr; e += NT) stf<T>(dst + e, out_s[e]);
+  for (int e = tid; e < R; e += NT) stf<T>(dst + kvr + e, turned(qr + D, e));
+}
+
+// out[t, h] = (a[t, h] uv[h]) * sigmoid(gate[t, h])  (gate null: 1).  LDS: a [R] | out [Dv] | shares [8 NT]
+template <typename T>
+__global__ void __launch_bounds__(NT) head_expand_gate_kernel(const T* __restrict__ a, const T* __restrict__ uv,
+                                                              const T* __restrict__ gate, int gate_ld, T* __restrict__ out,
+                                                              int H, int R, int Dv) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  float *x_s = smem, *out_s = smem + R, *red_s = smem + R + Dv;
+  const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  for (int r = tid; r < R; r += NT) x_s[r] = ldf<T>(a + ((size_t)t * H + h) * R + r);
+  __syncthreads();
+  vec_mat<T>(x_s, uv + (size_t)h * R * Dv, R, Dv, out_s, red_s);
+  for (int d = tid; d < Dv; d += NT) {
+    float v = out_s[d];
+    if (gate) v *= sigmoidf_(ldf<T>(gate + (size_t)t * gate_ld + h * Dv + d));
+    stf<T>(out + ((size_t)t * H + h) * Dv + d, v);
+  }
+}
+
+// out[t, h, d] = v[h, t, d] * sigmoid(gate[t, h Dv + d]): the batched product's layout back to rows, with the gate.
+// C = 8 (Dv, gate_ld multiples of 8, aligned) or 1 columns per thread.
+template <typename T, int C>
+__global__ void __launch_bounds__(NT) heads_gate_kernel(const T* __restrict__ v, const T* __restrict__ gate, int gate_ld,
+                                                        T* __restrict__ out, int rows, int H, int Dv) {
+  const size_t t = blockIdx.x;
+  const int HD = H * Dv;
+  for (int e = (blockIdx.y * NT + threadIdx.x) * C; e < HD; e += gridDim.y * NT * C) {
+    const int h = e / Dv, d = e % Dv;
+    const T* src = v + ((size_t)h * rows + t) * Dv + d;
+    if constexpr (C == 8) {
+      float a[8], g[8];
+      load8<T>(src, a);
+      load8<T>(gate + t * gate_ld + e, g);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] *= sigmoidf_(g[i]);
+      store8<T>(out + t * HD + e, a);
+    } else {
+      stf<T>(out + t * HD + e, ldf<T>(src) * sigmoidf_(ldf<T>(gate + t * gate_ld + e)));
+    }
+  }
+}
+
 // ---------------------------------------------------------------------------------- gated delta rule
 // prep row = q [G, N] | k [G, N] | decay [H, N] | beta [H], all fp32
 template <typename T>
@@ -265,15 +386,6 @@ __global__ void __launch_bounds__(NT) delta_prep_kernel(const T* __restrict__ qk
     pr[2 * GN + e] = expf(-expf(A_log[e / N]) * sp);
   }
   for (int e = tid; e < H; e += NT) pr[2 * GN + HN + e] = sigmoidf_(ldf<T>(u + t * ld + b0 + e));
-}
-
-// sum over the 16 lanes of a DPP row (quad swaps, then row rotations by 4 and 8); every lane gets the sum
-__device__ __forceinline__ float row16_sum(float v) {
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xF, 0xF, false));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xF, 0xF, false));
-  return v;
 }
 
 // GD = decay numbers per head in a prep row: N (one per key channel) or 1 (one for the head's whole state).
@@ -455,6 +567,73 @@ __global__ void __launch_bounds__(64) moe_topk_kernel(const float* __restrict__ 
   }
 }
 
+// One wave per token over its logits z [E + gate]: s = softmax over the experts, c = s + corr; a group (E / groups
+// neighbours) is as good as its best c, experts outside the `keep` best groups (the lower group on a tie) leave
+// the choice; the `top` largest c (the lower id on a tie) are chosen, weights s / (their sum + 1e-20) * scale.
+// gate_w: sigmoid of the last logit.  LDS: s [E] | c [E] | group scores [groups].
+__global__ void __launch_bounds__(64) route_grouped_kernel(const float* __restrict__ z, int E, int gate,
+                                                           const float* __restrict__ corr, int groups, int keep, int top,
+                                                           float scale, int* __restrict__ idx, float* __restrict__ wts,
+                                                           float* __restrict__ gate_w) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  float *s_s = smem, *c_s = smem + E, *g_s = smem + 2 * E;
+  const size_t t = blockIdx.x;
+  const int lane = threadIdx.x, size = E / groups;
+  const float* zr = z + t * (E + gate);
+  float mx = -INFINITY, sum = 0.f;
+  for (int e = lane; e < E; e += 64) { s_s[e] = zr[e]; mx = fmaxf(mx, s_s[e]); }
+  mx = wave_max(mx);
+  for (int e = lane; e < E; e += 64) sum += expf(s_s[e] - mx);
+  sum = wave_sum(sum);
+  for (int e = lane; e < E; e += 64) {
+    const float s = expf(s_s[e] - mx) / sum;
+    s_s[e] = s;
+    c_s[e] = s + (corr ? corr[e] : 0.f);
+  }
+  __syncthreads();
+  if (groups > 1) {
+    for (int g = lane; g < groups; g += 64) {
+      float b = -INFINITY;
+      for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, c_s[e]);
+      g_s[g] = b;
+    }
+    __syncthreads();
+    for (int g = lane; g < groups; g += 64) {
+      int better = 0;
+      for (int o = 0; o < groups; ++o) better += g_s[o] > g_s[g] || (g_s[o] == g_s[g] && o < g);
+      if (better >= keep)
+        for (int e = g * size; e < (g + 1) * size; ++e) c_s[e] = -INFINITY;
+    }
+    __syncthreads();
+  }
+  float tot = 0.f, my_w = 0.f;
+  int my_i = 0;                                              // lane k keeps the k-th choice
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY;
+    int bi = E;
+    for (int e = lane; e < E; e += 64)
+      if (c_s[e] > best) { best = c_s[e]; bi = e; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
+    }
+    if (bi >= E) bi = k;                                     // scores that compare with nothing (NaN): keep the ids in range
+    const float s = s_s[bi];
+    if (lane == k) { my_w = s; my_i = bi; }
+    tot += s;
+    __syncthreads();
+    if (lane == 0) c_s[bi] = -INFINITY;
+    __syncthreads();
+  }
+  if (lane < top) {
+    idx[t * top + lane] = my_i;
+    wts[t * top + lane] = my_w / (tot + 1e-20f) * scale;
+  }
+  if (gate && lane == 0) gate_w[t] = sigmoidf_(zr[E]);
+}
+
 // decode-sized steps: out row r of pair (token, choice) = act(gate_r . h, up_r . h); one wave per row at a time,
 // lanes stride the width with 8-element loads, the token's row sits in LDS as fp32.  silu: the activation is
 // silu(w gate) (w up) with w = in_w[pair] (null: 1), the unit of an input scaled by the router's weight.
@@ -519,6 +698,50 @@ __global__ void __launch_bounds__(NT) moe_down_kernel(const T* __restrict__ y, i
     }
     acc = wave_sum(acc);
     if (lane == 0) stf<T>(out + pair * W + r, acc);
+  }
+}
+
+// dot product of a weight row with a vector in LDS by one wave (every lane gets the sum)
+template <typename T>
+__device__ __forceinline__ float wave_dot(const T* __restrict__ w, const float* v_s, int n, int lane) {
+  float acc = 0.f;
+  if (n % 8 == 0) {
+#pragma unroll 2
+    for (int c = lane * 8; c < n; c += 64 * 8) {
+      float a[8];
+      load8<T>(w + c, a);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc += a[e] * v_s[c + e];
+    }
+  } else {
+    for (int c = lane; c < n; c += 64) acc += ldf<T>(w + c) * v_s[c];
+  }
+  return wave_sum(acc);
+}
+
+// Pairs p < rows * top are (token, choice) of the routed experts, pairs after them one per token of the shared
+// expert (own weights and width).  UP: y = max(W_up h, 0)^2;  else out = W_down y.
+template <typename T, bool UP>
+__global__ void __launch_bounds__(NT) relu2_experts_kernel(const T* __restrict__ in, const T* __restrict__ in_sh,
+                                                           const int* __restrict__ idx, int routed, int top,
+                                                           const T* __restrict__ w, const T* __restrict__ w_sh, int W, int ff,
+                                                           int sff, T* __restrict__ out, T* __restrict__ out_sh,
+                                                           int rows_per_wg, int E) {
+  extern __shared__ __attribute__((aligned(16))) float v_s[];
+  const int pair = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const bool sh = pair >= routed;
+  const int t = sh ? pair - routed : pair / top, f = sh ? sff : ff, K = UP ? W : f, R = UP ? f : W;
+  const int r0 = blockIdx.y * rows_per_wg, r1 = min(R, r0 + rows_per_wg);
+  if (r0 >= R) return;
+  const T* src = UP ? in + (size_t)t * W : sh ? in_sh + (size_t)t * sff : in + (size_t)pair * ff;
+  for (int c = tid; c < K; c += NT) v_s[c] = ldf<T>(src + c);
+  __syncthreads();
+  const T* wm = sh ? w_sh : w + (size_t)min(max(idx[pair], 0), E - 1) * ff * W;
+  T* dst = sh ? out_sh + (size_t)t * R : out + (size_t)pair * R;
+  for (int r = r0 + wave; r < r1; r += NT / 64) {
+    float v = wave_dot<T>(wm + (size_t)r * K, v_s, K, lane);
+    if constexpr (UP) { v = fmaxf(v, 0.f); v *= v; }
+    if (lane == 0) stf<T>(dst + r, v);
   }
 }
 
@@ -662,6 +885,78 @@ int edge_sm_moe_experts(const void* h, int W, const int* idx, int top, const voi
                                (const T*)h, W, idx, top, (const T*)w_gu, ff, limit, (T*)y, rpw, E, silu, in_w));
   SM_T(f32, hipLaunchKernelGGL(moe_down_kernel<T>, dim3(rows * top, (W + rpw - 1) / rpw), dim3(NT), (size_t)ff * 4, st,
                                (const T*)y, ff, idx, (const T*)w_down, W, (T*)out, rpw, E));
+  return (int)hipGetLastError();
+}
+
+// router: fp32 [E + gate, W]; z: fp32 scratch [rows, E + gate]
+int edge_sm_moe_route_grouped(const void* h, int W, const float* router, int E, int gate, const float* corr, int groups,
+                              int keep, int top, float scale, float* z, int* idx, float* wts, float* gate_w, int rows, int f32,
+                              hipStream_t st) {
+  if (rows == 0) return 0;
+  if (E < 1 || groups < 1 || E % groups || keep < 1 || keep > groups || top < 1 || top > 64 || top > E / groups * keep ||
+      E > 4096 || (gate && !gate_w))
+    return -2;
+  SM_T(f32, hipLaunchKernelGGL(moe_logits_kernel<T>, dim3(rows, (E + gate + NT / 64 - 1) / (NT / 64)), dim3(NT), 0, st,
+                               (const T*)h, W, router, E + gate, z, (const float*)nullptr));
+  hipLaunchKernelGGL(route_grouped_kernel, dim3(rows), dim3(64), (size_t)(2 * E + groups) * 4, st, (const float*)z, E, gate,
+                     corr, groups, keep, top, scale, idx, wts, gate_w);
+  return (int)hipGetLastError();
+}
+
+// w_up [E, ff, W], w_down [E, W, ff]; sff > 0: the shared expert su [sff, W], sd [W, sff].  Scratch y [rows * top, ff]
+// and ys [rows, sff]; out [rows * top, W], out_sh [rows, W]
+int edge_sm_moe_experts_relu2(const void* h, int W, const int* idx, int top, const void* w_up, const void* w_down, int ff,
+                              const void* su, const void* sd, int sff, void* y, void* ys, void* out, void* out_sh, int rows,
+                              int E, int f32, hipStream_t st) {
+  if (rows == 0) return 0;
+  if (ff < 1 || W < 1 || (sff > 0 && (!su || !sd || !ys || !out_sh))) return -2;
+  const int big = sff > ff ? sff : ff;
+  if ((size_t)W * 4 > 60 * 1024 || (size_t)big * 4 > 60 * 1024) return -3;
+  const int rpw = 16, routed = rows * top, pairs = routed + (sff > 0 ? rows : 0);
+  SM_T(f32, hipLaunchKernelGGL((relu2_experts_kernel<T, true>), dim3(pairs, (big + rpw - 1) / rpw), dim3(NT), (size_t)W * 4, st,
+                               (const T*)h, (const T*)h, idx, routed, top, (const T*)w_up, (const T*)su, W, ff, sff, (T*)y,
+                               (T*)ys, rpw, E));
+  SM_T(f32, hipLaunchKernelGGL((relu2_experts_kernel<T, false>), dim3(pairs, (W + rpw - 1) / rpw), dim3(NT), (size_t)big * 4,
+                               st, (const T*)y, (const T*)ys, idx, routed, top, (const T*)w_down, (const T*)sd, W, ff, sff,
+                               (T*)out, (T*)out_sh, rpw, E));
+  return (int)hipGetLastError();
+}
+
+int edge_sm_latent_expand_write(const void* u, int ld, int c0, const float* w, float eps, const void* q, const void* uk,
+                                const int* tok_seq, const int* tok_pos, const int* seq_slot, const int* ptab, int ptab_ld,
+                                const float* cs, void* pages, void* qc, int rows, int H, int D, int R, int kvr, int rot, int page,
+                                int f32, hipStream_t st) {
+  if (rows == 0) return 0;
+  if (rot % 2 || rot > R || (rot > 0 && !cs) || !u || !w) return -2;
+  const size_t lds = sizeof(float) * ((size_t)D + kvr + 8 * NT);
+  if (lds > 60 * 1024) return -3;
+  SM_T(f32, hipLaunchKernelGGL(latent_expand_write_kernel<T>, dim3(rows, H + 1), dim3(NT), lds, st, (const T*)u, ld, c0, w, eps,
+                               (const T*)q, (const T*)uk, tok_seq, tok_pos, seq_slot, ptab, ptab_ld, cs, (T*)pages, (T*)qc, H,
+                               D, R, kvr, rot, page));
+  return (int)hipGetLastError();
+}
+
+int edge_sm_head_expand_gate(const void* a, const void* uv, const void* gate, int gate_ld, void* out, int rows, int H, int R,
+                             int Dv, int f32, hipStream_t st) {
+  if (rows == 0) return 0;
+  const size_t lds = sizeof(float) * ((size_t)R + Dv + 8 * NT);
+  if (lds > 60 * 1024) return -3;
+  SM_T(f32, hipLaunchKernelGGL(head_expand_gate_kernel<T>, dim3(rows, H), dim3(NT), lds, st, (const T*)a, (const T*)uv,
+                               (const T*)gate, gate_ld, (T*)out, H, R, Dv));
+  return (int)hipGetLastError();
+}
+
+int edge_sm_heads_gate(const void* v, const void* gate, int gate_ld, void* out, int rows, int H, int Dv, int f32,
+                       hipStream_t st) {
+  if (rows == 0 || H * Dv == 0) return 0;
+  const bool vec = Dv % 8 == 0 && gate_ld % 8 == 0 && (((uintptr_t)v | (uintptr_t)gate | (uintptr_t)out) & 15) == 0;
+  const int per = NT * (vec ? 8 : 1), gy = (H * Dv + per - 1) / per < 8 ? (H * Dv + per - 1) / per : 8;
+  if (vec)
+    SM_T(f32, hipLaunchKernelGGL((heads_gate_kernel<T, 8>), dim3(rows, gy), dim3(NT), 0, st, (const T*)v, (const T*)gate,
+                                 gate_ld, (T*)out, rows, H, Dv));
+  else
+    SM_T(f32, hipLaunchKernelGGL((heads_gate_kernel<T, 1>), dim3(rows, gy), dim3(NT), 0, st, (const T*)v, (const T*)gate,
+                                 gate_ld, (T*)out, rows, H, Dv));
   return (int)hipGetLastError();
 }
 

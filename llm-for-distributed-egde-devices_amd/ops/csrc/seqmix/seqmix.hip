@@ -950,14 +950,6 @@ __global__ void __launch_bounds__(64) ssd_kernel(const T* __restrict__ xbc, int 
 // (1) every chunk's own contribution to its end state, all chunks in parallel; (2) the states at
 // the chunk borders, one short pass per sequence; (3) every chunk's outputs, all chunks in parallel.
 // All fp32 FMAs; every exponent is <= 0.
-constexpr int CL = 64;
-
-__device__ __forceinline__ int chunk_base(const int* __restrict__ seq_len, int s) {
-  int b = 0;
-  for (int i = 0; i < s; ++i) b += (seq_len[i] + CL - 1) / CL;
-  return b;
-}
-
 // step sizes and inclusive log-decay of one chunk into LDS (first wave; tc <= 64 tokens)
 template <typename T>
 __device__ __forceinline__ void chunk_steps(const T* __restrict__ u, int ld, int dt0, int h, float bias, float a,

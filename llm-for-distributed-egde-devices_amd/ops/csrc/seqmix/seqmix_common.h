@@ -35,4 +35,21 @@ __device__ __forceinline__ float siluf_(float x) { return x * sigmoidf_(x); }
 
 constexpr int NT = 256;
 
+// sum over the 16 lanes of a DPP row (quad swaps, then row rotations by 4 and 8); every lane gets the sum
+__device__ __forceinline__ float row16_sum(float v) {
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xF, 0xF, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xF, 0xF, false));
+  return v;
+}
+
+// chunked recurrences: tokens per chunk, and a sequence's first chunk among all chunks of the step
+constexpr int CL = 64;
+__device__ __forceinline__ int chunk_base(const int* __restrict__ seq_len, int s) {
+  int b = 0;
+  for (int i = 0; i < s; ++i) b += (seq_len[i] + CL - 1) / CL;
+  return b;
+}
+
 }  // namespace
