@@ -287,7 +287,7 @@ def test_embedding_with_learned_positions(dev):
 
 
 ROUTES = [  # experts, top, groups, keep, spread of the correction
-    (6, 2, 3, 2, 0.3), (16, 4, 4, 3, 0.05), (70, 5, 7, 1, 0.5), (8, 3, 1, 1, 0.2), (9, 9, 3, 3, 1.0), (130, 1, 65, 2, 2.0), (12, 6, 2, 1, 0.0)]
+    (6, 2, 3, 2, 0.3), (20, 4, 5, 3, 0.05), (70, 5, 7, 1, 0.5), (8, 3, 1, 1, 0.2), (9, 9, 3, 3, 1.0), (130, 1, 65, 2, 2.0), (12, 6, 2, 1, 0.0)]
 
 
 @pytest.mark.parametrize("dev", DEVS)
@@ -766,7 +766,7 @@ def test_graph_replays_against_eager_steps(tmp_path, precision):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("case", [(2, 64, 64, 16.0, 16, 1.0, (500, 65)), (2, 48, 32, 4.0, 8, 2.0, (131, 1)), (1, 128, 128, 16.0, 16, 3.0, (300, 2)),
+@pytest.mark.parametrize("case", [(2, 64, 64, 16.0, 16, 1.0, (500, 65)), (2, 40, 32, 4.0, 8, 2.0, (131, 1)), (1, 128, 128, 16.0, 16, 3.0, (300, 2)),
                                   (3, 20, 136, 1.0, 4, 0.0, (100, 33))])
 def test_bf16_linear_attention_in_both_forms(case):
     """bf16 inputs: the chunked and the token-by-token kernels against float64 on the same rounded projections."""
