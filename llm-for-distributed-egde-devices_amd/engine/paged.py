@@ -17,7 +17,8 @@ Per run:
       shared key part; a layer that reads another layer's cache holds the same tensor as that run
   canon1 / canon2 [slots, taps - 1, width] fp32                 last inputs of the sublayers' input convolutions
   k = v [pages, page, kv heads, D]                              attention whose values are its keys: one tensor
-  k, v as in the first line for gated attention (the values are cached turned by their position)
+  k, v as in the first line for gated attention (the values are cached turned by their position, where the
+      design turns them), alone or beside a linear attention's ssm
 and, for models whose embedding looks at the previous token, ``prev_tok`` int64 [slots].
 A slot's recurrent rows are not cleared on release: a portion that starts at position 0 ignores
 what the slot held (the kernels start from zero there).
@@ -69,8 +70,9 @@ class PagedCache:
                     d = delta
                     rc.conv = torch.zeros(slots, max(d.conv - 1, 1), d.conv_channels, dtype=dtype, device=device)
                     rc.ssm = torch.zeros(slots, d.heads, d.dim, d.vdim, dtype=torch.float32, device=device)
-                elif getattr(s, "gla", None) is not None:
-                    rc.ssm = torch.zeros(slots, s.gla.heads, s.gla.dim, s.gla.vdim, dtype=torch.float32, device=device)
+                linear = getattr(s, "gla", None) or getattr(s, "decay_attn", None)
+                if linear is not None:                     # alone or beside the attention's pages
+                    rc.ssm = torch.zeros(slots, linear.heads, linear.dim, linear.vdim, dtype=torch.float32, device=device)
                 if canon_taps:
                     rc.canon1 = torch.zeros(slots, max(canon_taps - 1, 1), width, dtype=torch.float32, device=device)
                     if getattr(s, "moe", None) is not None or getattr(s, "ff", None):

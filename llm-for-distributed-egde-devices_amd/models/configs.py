@@ -19,7 +19,10 @@ Families (dims are public HF configs):
                            grouped-query attention with rotated values, both with a window and a sink,
                            PolyNorm and mixture-of-experts feed-forwards, several residual streams) and
                            Numizen (gated latent attention and gated linear attention beside a gelu-gated
-                           or group-limited expert feed-forward, Dynamic Tanh norms, learned positions)
+                           or group-limited expert feed-forward, Dynamic Tanh norms, learned positions) and
+                           Felavik (gated attention with a bucketed distance bias side by side with
+                           retention, lightning attention, group-limited silu-gated experts, layers that
+                           run on another layer's weights)
 A single ``ModelConfig`` describes all decoder families; ``DecoderLM`` interprets the flags.
 """
 from __future__ import annotations
@@ -153,7 +156,10 @@ class GatedAttnSpec:
     times a learned number per head (``temp``); a sliding window of ``window`` positions beside the
     first ``keep_first`` tokens of the sequence, which stay visible at their own positions; exp(sink_h)
     in the softmax denominator (``sink``); the concatenated heads times sigmoid(W_g h), element by
-    element (``gate``)."""
+    element (``gate``); a bias on the q, k and v projections (``qkv_bias``); q times
+    1 + coef ln(floor((position + 1) / every) + 1) (``q_temp`` = (coef, every)); a learned number per head
+    and bucket of the distance n = i - j, added to the scaled score (``rel_buckets`` rows B, ``rel_max`` D:
+    row n below B/2, then B/2 + floor(ln(n / (B/2)) / ln(D / (B/2)) (B - B/2)), at most B - 1)."""
     heads: int
     kv_heads: int
     dim: int
@@ -169,6 +175,10 @@ class GatedAttnSpec:
     temp: bool = True
     sink: bool = True
     gate: bool = True
+    qkv_bias: bool = False
+    q_temp: Optional[tuple] = None       # (coef, every)
+    rel_buckets: int = 0
+    rel_max: int = 0
 
     @property
     def proj_sizes(self):
@@ -228,6 +238,31 @@ class GLASpec:
 
 
 @dataclass
+class DecayAttnSpec:
+    """Linear attention with one fixed decay per head: S <- decay_h S + k v^T over a [dim, vdim] fp32 state,
+    o = S^T q, no denominator.  ``act`` "silu": q, k and v pass through silu after their projections ("none": as
+    they are); rotary positions on the first ``rot_dims`` coordinates of q and k, coordinate i paired with
+    i + rot_dims / 2 (0: none); k times ``k_scale`` after the rotation.  ``norm`` "head": each head's o over its own
+    root mean square, no weight; "all": the concatenated heads over their common root mean square, with a weight
+    vector.  Then times silu or sigmoid (``gate_act``) of W_g h."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    act: str = "none"
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    k_scale: float = 1.0
+    norm: str = "head"
+    gate_act: str = "silu"
+
+    @property
+    def in_sizes(self):
+        """Row blocks of the fused input projection: q | k | v | gate."""
+        return (self.heads * self.dim, self.heads * self.dim, self.heads * self.vdim, self.heads * self.vdim)
+
+
+@dataclass
 class MoESpec:
     """Mixture of gated-linear experts.  ``router`` "softmax": softmax over ``experts``, the ``top``
     largest renormalised and multiplied by ``scale``; "sigmoid": scores sigmoid(W_r h), the ``top``
@@ -272,6 +307,8 @@ class LayerSpec:
                                              # one mixer, a norm before each sublayer, several residual streams
                                              # "gla" (and "latent_attention" in a model whose mixer and feed-forward run
                                              # side by side behind their own norms)
+                                             # "attention_retention" (``gated_attn`` and ``decay_attn`` side by side, each
+                                             # times its scale) and "lightning" (``decay_attn`` alone)
     attn: Optional[WindowAttnSpec] = None
     ssd: Optional[SSDSpec] = None
     ff: Optional[int] = None
@@ -283,6 +320,10 @@ class LayerSpec:
     chunk_attn: Optional[ChunkAttnSpec] = None
     gated_attn: Optional[GatedAttnSpec] = None
     gla: Optional[GLASpec] = None
+    decay_attn: Optional[DecayAttnSpec] = None
+    left_scale: float = 1.0                  # "attention_retention": the weights of the two sides in their sum
+    right_scale: float = 1.0
+    weights_of: Optional[int] = None         # the layer whose weights this one runs on (its cache and state are its own)
 
 
 @dataclass
@@ -348,12 +389,21 @@ class ModelConfig:
     # is added to the embedding; no sequence may grow past ``max_position_embeddings``), ``layer_scale`` (each
     # sublayer's result times a vector before the sum)
     layer_scale: bool = False
+    # arch "felavik": ``logit_softcap`` tanh(logits / ``logit_softcap``)
+    logit_softcap: Optional[float] = None
+
+    def weight_layer(self, i: int) -> int:
+        """The layer whose weights layer i runs on (itself, unless its spec names another)."""
+        while self.layer_specs is not None and self.layer_specs[i].weights_of is not None:
+            i = self.layer_specs[i].weights_of
+        return i
 
     def layer_runs(self) -> List[tuple]:
-        """[(layer index, pass number or None)] in execution order; every run has its own cache."""
+        """[(layer index, pass number or None)] in execution order; every run has its own cache.  A layer without
+        weights of its own runs as the layer it shares them with (``weight_layer``)."""
         n = self.num_layers
         if self.loop is None:
-            return [(i, None) for i in range(n)]
+            return [(self.weight_layer(i), None) for i in range(n)]
         lp = self.loop
         runs = [(i, None) for i in range(lp.start)]
         for t in range(lp.times):
@@ -532,7 +582,7 @@ def checkpoint_shapes(path: str) -> dict:
 def from_hf_dir(path: str) -> ModelConfig:
     with open(os.path.join(path, "config.json")) as f:
         c = json.load(f)
-    needs_shapes = str(c.get("architecture", "")).lower() in ("pagonex", "fikupel", "numizen")
+    needs_shapes = str(c.get("architecture", "")).lower() in ("pagonex", "fikupel", "numizen", "felavik")
     return from_hf_config(c, checkpoint_shapes(path) if needs_shapes else None)
 
 
@@ -945,6 +995,102 @@ def to_numizen_config(cfg: ModelConfig) -> dict:
     return out
 
 
+def from_felavik_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
+    """The Felavik layout of ``config.json``: ``layers`` (``type`` = ``parallel`` or ``lightning``, ``mixer`` sizes and
+    constants, ``mlp`` = mixture of experts or null, ``weights_of`` = the layer whose tensors serve this one),
+    ``embedding.scale``, ``logit_softcap``, ``norm.eps``, ``vocab``, ``width``.  ``shapes`` (tensor name -> shape of
+    the checkpoint) supplies the number of distance buckets."""
+    n, specs = len(c["layers"]), []
+    for i, l in enumerate(c["layers"]):
+        m, kind = l["mixer"], l["type"]
+        of, own = l.get("weights_of"), i
+        for _ in range(n):
+            if c["layers"][own].get("weights_of") is None:
+                break
+            own = int(c["layers"][own]["weights_of"])
+            if not 0 <= own < n:
+                raise ValueError(f"layer {i}: weights_of names no layer")
+        else:
+            raise ValueError(f"layer {i}: weights_of goes round in a circle")
+        if (c["layers"][own]["type"], c["layers"][own]["mixer"], c["layers"][own].get("mlp")) != (kind, m, l.get("mlp")):
+            raise ValueError(f"layer {i} differs from the layer whose weights it runs on")
+        ga, ls, rs = None, 1.0, 1.0
+        if kind == "parallel":
+            a, r, ls, rs = m["left"], m["right"], float(m["left_scale"]), float(m["right_scale"])
+            t, rot = a.get("q_temp") or None, r.get("rot") or None
+            buckets = int(shapes[f"l{own}.mix.left.rel"][0]) if shapes is not None else int(a.get("rel_buckets", 32))
+            ga = GatedAttnSpec(heads=int(a["heads"]), kv_heads=int(a.get("kv_heads", a["heads"])), dim=int(a["dim"]),
+                               vdim=int(a["vdim"]), scale=float(a["scale"]), rotate_values=False, temp=False, sink=False,
+                               qkv_bias=True, q_temp=(float(t["coef"]), int(t["every"])) if t else None,
+                               rel_buckets=buckets, rel_max=int(a["bias_max"]))
+            if ga.heads % ga.kv_heads:
+                raise ValueError("heads must be a multiple of kv_heads")
+            if buckets < 2 or ga.rel_max <= buckets // 2:
+                raise ValueError("the distance bias needs two rows and a last bucket beyond the first half of them")
+            da = DecayAttnSpec(heads=int(r["heads"]), dim=int(r["dim"]), vdim=int(r["vdim"]), decay=tuple(map(float, r["decay"])),
+                               rot_dims=int(rot["dims"]) if rot else 0, rot_base=float(rot["base"]) if rot else 10000.0,
+                               k_scale=int(r["dim"]) ** -0.5)
+        elif kind == "lightning":
+            da = DecayAttnSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), decay=tuple(map(float, m["decay"])),
+                               act="silu", norm="all", gate_act="sigmoid")
+        else:
+            raise ValueError(f"unsupported layer type {kind!r}")
+        if len(da.decay) != da.heads or not all(0.0 <= d <= 1.0 for d in da.decay):
+            raise ValueError("one decay between 0 and 1 per head")
+        if da.rot_dims % 2 or da.rot_dims > da.dim:
+            raise ValueError("rotation runs over pairs of coordinates inside a head")
+        mlp, moe = l.get("mlp") or None, None
+        if mlp and mlp.get("kind", "moe") == "moe":
+            r, g = mlp["router"], mlp["router"].get("groups") or {}
+            moe = MoESpec(experts=int(r["experts"]), top=int(r["top"]), scale=1.0, ff=int(mlp["expert"]["ff"]), act="silu_glu",
+                          groups=int(g.get("count", 1)), groups_keep=int(g.get("keep", 1)))
+            if moe.experts % moe.groups or not 1 <= moe.groups_keep <= moe.groups:
+                raise ValueError("the experts must split into equal groups of which at least one is kept")
+            if not 1 <= moe.top <= moe.experts // moe.groups * moe.groups_keep:
+                raise ValueError("the kept groups hold fewer experts than a token uses")
+        elif mlp:
+            raise ValueError(f"unsupported feed-forward kind {mlp.get('kind')!r}")
+        specs.append(LayerSpec("attention_retention" if ga else "lightning", moe=moe, gated_attn=ga, decay_attn=da, left_scale=ls,
+                               right_scale=rs, weights_of=int(of) if of is not None else None))
+    first = specs[0].gated_attn or specs[0].decay_attn
+    cap = c.get("logit_softcap")
+    return ModelConfig(arch="felavik", vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), num_layers=n,
+                       num_heads=first.heads, num_kv_heads=getattr(first, "kv_heads", first.heads), intermediate_size=0,
+                       head_dim=first.dim, max_position_embeddings=1 << 20, norm="rms", norm_eps=float(c["norm"]["eps"]),
+                       act="silu_glu", pos_emb="rope", name=c.get("name", "felavik"), layer_specs=specs, streams=1, hyper=False,
+                       embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
+                       logit_softcap=float(cap) if cap else None)
+
+
+def to_felavik_config(cfg: ModelConfig) -> dict:
+    """Inverse of ``from_felavik_config`` (the number of distance buckets travels as a tensor shape)."""
+    layers = []
+    for s in cfg.layer_specs:
+        d = s.decay_attn
+        m = {"heads": d.heads, "dim": d.dim, "vdim": d.vdim, "decay": list(d.decay)}
+        if s.gated_attn is not None:
+            a = s.gated_attn
+            left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale, "bias_max": a.rel_max}
+            if a.q_temp:
+                left["q_temp"] = {"coef": a.q_temp[0], "every": a.q_temp[1]}
+            if d.rot_dims:
+                m["rot"] = {"dims": d.rot_dims, "base": d.rot_base}
+            m = {"left": left, "right": m, "left_scale": s.left_scale, "right_scale": s.right_scale}
+        mlp = None
+        if s.moe is not None:
+            e = s.moe
+            mlp = {"kind": "moe", "router": {"experts": e.experts, "top": e.top, "groups": {"count": e.groups, "keep": e.groups_keep}},
+                   "expert": {"ff": e.ff}}
+        layers.append({"type": "parallel" if s.gated_attn is not None else "lightning", "mixer": m, "mlp": mlp})
+        if s.weights_of is not None:
+            layers[-1]["weights_of"] = s.weights_of
+    out = {"architecture": "Felavik", "vocab": cfg.vocab_size, "width": cfg.hidden_size, "layers": layers,
+           "norm": {"eps": cfg.norm_eps}, "embedding": {"scale": cfg.embed_scale}}
+    if cfg.logit_softcap is not None:
+        out["logit_softcap"] = cfg.logit_softcap
+    return out
+
+
 def from_hf_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
     """Map a ``config.json`` onto ModelConfig (Hugging Face ``model_type`` layouts, or an
     ``architecture`` key naming a per-layer layout; ``shapes``: the checkpoint's tensor shapes, for
@@ -959,6 +1105,8 @@ def from_hf_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
         return from_fikupel_config(c, shapes)
     if str(c.get("architecture", "")).lower() == "numizen":
         return from_numizen_config(c, shapes)
+    if str(c.get("architecture", "")).lower() == "felavik":
+        return from_felavik_config(c, shapes)
     mt = c.get("model_type")
     eos = c.get("eos_token_id")
     if isinstance(eos, list):

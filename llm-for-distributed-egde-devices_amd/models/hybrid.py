@@ -1,4 +1,4 @@
-"""Layer-spec language models (arch "nudadra", "pagonex", "vetevik", "fikupel", "numizen"): every layer is
+"""Layer-spec language models (arch "nudadra", "pagonex", "vetevik", "fikupel", "numizen", "felavik"): every layer is
 described by its own entry of ``ModelConfig.layer_specs``, a span of layers may run several times in a row,
 and the residual stream is fp32.
 
@@ -20,7 +20,10 @@ u = sum_s a_s x_s, computes y = f(RMSnorm(u)), and every stream becomes x_r <- s
 (a, M, b learned per sublayer); with one stream and no such weights this is x <- x + f(norm(x)).  The
 mixer is latent attention without positions or gated grouped-query attention, the feed-forward a
 PolyNorm unit or a mixture of experts; the final norm reads the sum of the streams and the embedding
-table is the output projection.
+table is the output projection.  With one stream the mixer may also be gated attention side by side with
+retention, or linear attention with fixed decays ("felavik"): the feed-forward is a mixture of silu-gated
+experts limited to groups, a layer may run on another layer's weights with a cache of its own, and the
+logits are capped as c tanh(z / c).
 
 Per layer (side by side behind two norms, ``TwoNormLayer``):  x <- x + s1 mixer(N1(x)) + s2 ff(N2(x)), both of the
 same x, every N a Dynamic Tanh (tanh(alpha x) w + b) and s1, s2 learned vectors.  The mixer is latent attention
@@ -51,8 +54,8 @@ import torch.nn as nn
 from ..ops import seqmix
 from .configs import LayerSpec, ModelConfig
 from .layers import DynamicTanh, GroupRMSNorm, Linear, RowLayerNorm, ScalarNorm
-from .mixers import (ChannelDeltaMixer, ChunkAttention, GatedAttention, GatedLinearAttention, HeadDeltaMixer,
-                     LatentAttention, ParallelMixer)
+from .mixers import (AttentionRetention, ChannelDeltaMixer, ChunkAttention, DecayLinearAttention, GatedAttention,
+                     GatedLinearAttention, HeadDeltaMixer, LatentAttention, ParallelMixer)
 from .moe import MoEFeedForward, MoEOut
 
 
@@ -180,8 +183,8 @@ class PolyNormFF(nn.Module):
 
 
 class HyperLayer(nn.Module):
-    """One mixer (latent attention without positions or gated attention) and an optional feed-forward
-    (PolyNorm unit or mixture of experts), each reading the RMS norm of a weighted sum of the residual
+    """One mixer (latent attention without positions, gated attention, gated attention beside retention, or linear
+    attention with fixed decays) and an optional feed-forward (PolyNorm unit or mixture of experts), each reading the RMS norm of a weighted sum of the residual
     streams and written back into all of them; one stream without weights: the plain pre-norm residual."""
 
     def __init__(self, cfg: ModelConfig, spec: LayerSpec, idx: int, dtype, device):
@@ -192,6 +195,10 @@ class HyperLayer(nn.Module):
             self.mix = LatentAttention(spec.latent, W, eps, dtype, device)
         elif spec.mixer == "gated_attention":
             self.mix = GatedAttention(spec.gated_attn, W, eps, dtype, device)
+        elif spec.mixer == "attention_retention":
+            self.mix = AttentionRetention(spec, W, eps, dtype, device)
+        elif spec.mixer == "lightning":
+            self.mix = DecayLinearAttention(spec.decay_attn, W, eps, dtype, device)
         else:
             raise ValueError(spec.mixer)
         self.norm1 = StreamNorm(W, eps, device)
@@ -230,14 +237,15 @@ class HyperLayer(nn.Module):
         hc = self.hc2
         h = seqmix.hyper_update(X, mix, out, y, nxt=(hc.inp if hc is not None else None, self.norm2.weight, self.norm2.eps))
         mix, out = (hc.mix, hc.out) if hc is not None else (None, None)
-        if self.spec.moe is not None:
-            shared, parts, wts = self.ff(h)
+        if self.spec.moe is None:
+            f = MoEOut(self.ff(h), None, None, None, None)
+        elif self.spec.moe.router == "softmax":
+            f = self.ff.run(h)
         else:
-            shared, parts, wts = self.ff(h), None, None
-        if nxt is not None:
-            return X, seqmix.hyper_update(X, mix, out, shared, parts, wts, nxt=nxt)
-        seqmix.hyper_update(X, mix, out, shared, parts, wts)
-        return X, None
+            shared, parts, wts = self.ff(h)
+            f = MoEOut(shared, None, parts, wts, None)
+        r = seqmix.hyper_update(X, mix, out, f.shared, f.parts, f.wts, nxt, f.rows)
+        return X, (r if nxt is not None else None)
 
 
 class GeluGLUFF(nn.Module):
@@ -319,7 +327,9 @@ class HybridLM(nn.Module):
         self.first, self.last = 0, cfg.num_layers
         self.has_embed = self.has_head = True
         self.embed = nn.Parameter(torch.empty(cfg.vocab_size, W, dtype=dtype, device=device), requires_grad=False)
-        self.layers = nn.ModuleList([_make_layer(cfg, s, i, dtype, device) for i, s in enumerate(cfg.layer_specs)])
+        # a layer that runs on another one's weights has no module of its own: ``runs`` names the other
+        self.layers = nn.ModuleList([_make_layer(cfg, s, i, dtype, device) if s.weights_of is None else nn.Identity()
+                                     for i, s in enumerate(cfg.layer_specs)])
         self.runs = cfg.layer_runs()
         if cfg.pos_emb == "learned":
             self.pos = nn.Parameter(torch.empty(cfg.max_position_embeddings, W, dtype=dtype, device=device), requires_grad=False)
@@ -398,7 +408,10 @@ class HybridLM(nn.Module):
                 return torch.empty(0, cfg.vocab_size, dtype=torch.float32, device=x.device)
             x = x.index_select(0, rows)
         h = self.final_norm(x, None, self.dtype) if cfg.streams else self.final_norm(x, self.dtype)
-        logits = self.lm_head(h).float()
+        logits = self.lm_head(h)
+        if cfg.logit_softcap is not None:
+            return seqmix.softcap(logits, cfg.logit_softcap)
+        logits = logits.float()
         return logits if cfg.logit_scale == 1.0 else logits.mul_(cfg.logit_scale)
 
 
@@ -796,11 +809,77 @@ def export_numizen_tensors(model: "HybridLM") -> Dict[str, torch.Tensor]:
     return {k: v.reshape(()) if k.endswith(".alpha") else v for k, v in out.items()}
 
 
+def _felavik_norms(i: int, spec: LayerSpec) -> list:
+    return [(f"layers.{i}.norm{n}.weight", f"l{i}.norm{n}") for n in (("1", "2") if spec.moe is not None else ("1",))]
+
+
+_FELAVIK_TOP = [("embed", "embed"), ("final_norm.weight", "final.norm"), ("lm_head.weight", "head")]
+
+
+def convert_felavik_tensors(cfg: ModelConfig, t: Dict[str, torch.Tensor]) -> Dict[str, torch.Tensor]:
+    """Checkpoint names of the Felavik layout (``l<i>.mix.left.q``, ``l<i>.mix.right.g``, ``l<i>.mlp.e<k>.gate`` ...) ->
+    this package's parameter names: one fused input and one fused output projection for both sides of a parallel
+    mixer, the biases in one row, stacked expert weights.  Layers that run on another one's weights have no tensors."""
+    out = {ours: t[theirs] for ours, theirs in _FELAVIK_TOP}
+    for i, spec in enumerate(cfg.layer_specs):
+        if spec.weights_of is not None:
+            continue
+        out.update({ours: t[theirs] for ours, theirs in _felavik_norms(i, spec)})
+        M, m = f"l{i}.mix.", f"layers.{i}.mix."
+        qkvg = ("q", "k", "v", "g")
+        if spec.gated_attn is not None:
+            L, R = M + "left.", M + "right."
+            out[m + "proj_in.weight"] = torch.cat([t[L + n] for n in qkvg] + [t[R + n] for n in qkvg], 0)
+            out[m + "left.qkv_b"] = torch.cat([t[L + n + ".b"] for n in qkvg[:3]], 0)
+            out[m + "left.q_norm"], out[m + "left.k_norm"], out[m + "left.rel"] = t[L + "q.norm"], t[L + "k.norm"], t[L + "rel"]
+            out[m + "o.weight"] = torch.cat([t[L + "o"], t[R + "o"]], 1)
+        else:
+            out[m + "proj_in.weight"] = torch.cat([t[M + n] for n in qkvg], 0)
+            out[m + "norm_w"], out[m + "o.weight"] = t[M + "norm"], t[M + "o"]
+        if spec.moe is not None:
+            e, F_, f = spec.moe, f"l{i}.mlp.", f"layers.{i}.ff."
+            out[f + "router"] = t[F_ + "router"]
+            out[f + "w_gu"] = torch.stack([torch.cat([t[f"{F_}e{k}.gate"], t[f"{F_}e{k}.up"]], 0) for k in range(e.experts)])
+            out[f + "w_down"] = torch.stack([t[f"{F_}e{k}.down"] for k in range(e.experts)])
+    return out
+
+
+def export_felavik_tensors(model: "HybridLM") -> Dict[str, torch.Tensor]:
+    """Inverse of ``convert_felavik_tensors`` (checkpoint names, 16-bit storage)."""
+    cfg = model.cfg
+    p = {k: v.detach() for k, v in model.named_parameters()}
+    out = {theirs: p[ours] for ours, theirs in _FELAVIK_TOP}
+    for i, spec in enumerate(cfg.layer_specs):
+        if spec.weights_of is not None:
+            continue
+        out.update({theirs: p[ours] for ours, theirs in _felavik_norms(i, spec)})
+        M, m = f"l{i}.mix.", f"layers.{i}.mix."
+        w, d = p[m + "proj_in.weight"], spec.decay_attn
+        if spec.gated_attn is not None:
+            a, L, R = spec.gated_attn, M + "left.", M + "right."
+            names = [L + n for n in ("q", "k", "v", "g")] + [R + n for n in ("q", "k", "v", "g")]
+            out.update(zip(names, torch.split(w, list(a.proj_sizes) + list(d.in_sizes), 0)))
+            out.update(zip([L + n + ".b" for n in ("q", "k", "v")], torch.split(p[m + "left.qkv_b"], list(a.proj_sizes[:3]), 0)))
+            out[L + "q.norm"], out[L + "k.norm"], out[L + "rel"] = p[m + "left.q_norm"], p[m + "left.k_norm"], p[m + "left.rel"]
+            out[L + "o"], out[R + "o"] = torch.split(p[m + "o.weight"], [a.heads * a.vdim, d.heads * d.vdim], 1)
+        else:
+            out.update(zip([M + n for n in ("q", "k", "v", "g")], torch.split(w, list(d.in_sizes), 0)))
+            out[M + "norm"], out[M + "o"] = p[m + "norm_w"], p[m + "o.weight"]
+        if spec.moe is not None:
+            e, F_, f = spec.moe, f"l{i}.mlp.", f"layers.{i}.ff."
+            out[F_ + "router"] = p[f + "router"]
+            for k in range(e.experts):
+                out[f"{F_}e{k}.gate"], out[f"{F_}e{k}.up"] = p[f + "w_gu"][k, :e.ff], p[f + "w_gu"][k, e.ff:]
+                out[f"{F_}e{k}.down"] = p[f + "w_down"][k]
+    return {k: v.to(torch.bfloat16).contiguous() for k, v in out.items()}
+
+
 CONVERTERS = {"nudadra": (convert_nudadra_tensors, export_nudadra_tensors),
               "pagonex": (convert_pagonex_tensors, export_pagonex_tensors),
               "vetevik": (convert_vetevik_tensors, export_vetevik_tensors),
               "fikupel": (convert_fikupel_tensors, export_fikupel_tensors),
-              "numizen": (convert_numizen_tensors, export_numizen_tensors)}
+              "numizen": (convert_numizen_tensors, export_numizen_tensors),
+              "felavik": (convert_felavik_tensors, export_felavik_tensors)}
 
 
 @torch.no_grad()
@@ -870,7 +949,7 @@ def init_random_hybrid_(model: HybridLM, seed: int = 0) -> HybridLM:
             v = 2.0 + r(*p.shape)
         elif leaf == "correction":
             v = 0.02 * r(*p.shape)
-        elif leaf == "router_b":
+        elif leaf in ("router_b", "rel"):
             v = 0.5 * r(*p.shape)
         elif leaf == "sink":
             v = r(*p.shape)

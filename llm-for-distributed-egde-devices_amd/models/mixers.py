@@ -16,7 +16,7 @@ import torch
 import torch.nn as nn
 
 from ..ops import seqmix
-from .configs import ChunkAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, SSDSpec, WindowAttnSpec
+from .configs import ChunkAttnSpec, DecayAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, LayerSpec, SSDSpec, WindowAttnSpec
 from .layers import Linear
 
 
@@ -196,35 +196,111 @@ class GatedAttention(nn.Module):
     """Grouped-query attention with an RMS norm per head on q and k, rotary positions on part of each
     head (neighbouring coordinates paired), values cached turned by their own position and each head's
     output turned back by the query's, a learned temperature and a learned sink per head, a sliding
-    window beside the sequence's first tokens, and an element-wise sigmoid gate from the same input.
-    One fused GEMM produces q | k | v | gate; the temperature is folded into q in fp32."""
+    window beside the sequence's first tokens, and an element-wise sigmoid gate from the same input; or
+    without rotation: biases on q, k and v, a temperature that grows with the position and a learned bias per
+    bucket of distances.  One fused GEMM produces q | k | v | gate; temperatures are folded into q in fp32.
+    ``inner``: the input and output projections belong to the module around it (``attend`` alone is used)."""
 
-    def __init__(self, spec: GatedAttnSpec, width: int, eps: float, dtype, device):
+    def __init__(self, spec: GatedAttnSpec, width: int, eps: float, dtype, device, inner: bool = False):
         super().__init__()
         self.spec, self.eps = spec, eps
         s = spec
         P = lambda *shape: nn.Parameter(torch.zeros(*shape, dtype=torch.float32, device=device), requires_grad=False)
-        self.proj_in = Linear(width, sum(s.proj_sizes), False, dtype, device)
+        self.proj_in = None if inner else Linear(width, sum(s.proj_sizes), False, dtype, device)
         self.q_norm = P(s.dim) if s.qk_norm else None
         self.k_norm = P(s.dim) if s.qk_norm else None
         self.temp = P(s.heads) if s.temp else None
         self.sink = P(s.heads) if s.sink else None
-        self.o = Linear(s.heads * s.vdim, width, False, dtype, device)
+        self.qkv_b = P(sum(s.proj_sizes[:3])) if s.qkv_bias else None
+        self.rel = P(s.rel_buckets, s.heads) if s.rel_buckets else None
+        self.o = None if inner else Linear(s.heads * s.vdim, width, False, dtype, device)
         self._rope, self._vrope = {}, {}
+        self._by_distance = (None, None)
 
-    def forward(self, h: torch.Tensor, meta: seqmix.RaggedMeta, run) -> torch.Tensor:
+    def by_distance(self) -> Optional[torch.Tensor]:
+        """The distance bias laid out by distance [heads, n], rebuilt when the learned table changes."""
+        if self.rel is None:
+            return None
+        key = (self.rel._version, self.rel.data_ptr())
+        if self._by_distance[0] != key:
+            self._by_distance = (key, seqmix.distance_bias_table(self.rel, self.spec.rel_max))
+        return self._by_distance[1]
+
+    def attend(self, u: torch.Tensor, c0: int, meta: seqmix.RaggedMeta, run, out: Optional[torch.Tensor] = None,
+               out_scale: float = 1.0) -> torch.Tensor:
+        """``u`` columns [c0, ..) hold q | k | v | gate.  Returns the gated heads [T, heads vdim], times ``out_scale``
+        and in ``out`` when that is given."""
         s = self.spec
         nq, nk, nv, ng = s.proj_sizes
-        u = self.proj_in(h)
-        rope = _shared_rope(self._rope, (s.rot_dims, s.rot_base, s.rot_scaling), meta.max_keys, h.device)
-        vrope = _shared_rope(self._vrope, (s.vdim, s.rot_base, None), meta.max_keys, h.device) if s.rotate_values else None
+        u = u[:, c0:c0 + nq + nk + nv + ng]
+        gate = u[:, nq + nk + nv:] if ng else None
+        rope = _shared_rope(self._rope, (s.rot_dims, s.rot_base, s.rot_scaling), meta.max_keys, u.device)
+        vrope = _shared_rope(self._vrope, (s.vdim, s.rot_base, None), meta.max_keys, u.device) if s.rotate_values else None
         q = seqmix.qk_norm_rope_write(u, meta, self.q_norm, self.k_norm, self.eps, rope, vrope, self.temp, run.k, run.v,
-                                      s.heads, s.rot_dims)
-        a = seqmix.window_pool_attention(q, None, run.k, run.v, None, None, meta, s.scale, s.window, None, self.sink,
-                                         s.keep_first)
-        if vrope is not None or ng:
-            a = seqmix.unrotate_gate(a, u[:, nq + nk + nv:nq + nk + nv + ng] if ng else None, meta, vrope, s.heads)
-        return self.o(a)
+                                      s.heads, s.rot_dims, self.qkv_b, s.q_temp)
+        attend = lambda g, o, sc: seqmix.window_pool_attention(q, g, run.k, run.v, None, None, meta, s.scale, s.window, None,
+                                                               self.sink, s.keep_first, self.by_distance(), o, sc)
+        if vrope is None:
+            return attend(gate, out, out_scale)
+        assert out is None and out_scale == 1.0
+        return seqmix.unrotate_gate(attend(None, None, 1.0), gate, meta, vrope, s.heads)
+
+    def forward(self, h: torch.Tensor, meta: seqmix.RaggedMeta, run) -> torch.Tensor:
+        return self.o(self.attend(self.proj_in(h), 0, meta, run))
+
+
+class DecayLinearAttention(nn.Module):
+    """Linear attention with one fixed decay per head (``DecayAttnSpec``: retention with rotated q and k and a norm
+    per head, or silu inputs and one norm over the heads): S <- decay_h S + k v^T and o = S^T q over a [dim, vdim]
+    fp32 state, the norm, a gate.  One fused GEMM produces q | k | v | gate.  ``inner``: the projections belong to the
+    module around it."""
+
+    def __init__(self, spec: DecayAttnSpec, width: int, eps: float, dtype, device, inner: bool = False):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        s = spec
+        self.proj_in = None if inner else Linear(width, sum(s.in_sizes), False, dtype, device)
+        self.register_buffer("decay", seqmix.decay_table(s.decay, device), persistent=False)
+        self.norm_w = nn.Parameter(torch.ones(s.heads * s.vdim, dtype=torch.float32, device=device), requires_grad=False) \
+            if s.norm == "all" else None
+        self.o = None if inner else Linear(s.heads * s.vdim, width, False, dtype, device)
+        self._rope = {}
+
+    def attend(self, u: torch.Tensor, c0: int, meta: seqmix.RaggedMeta, run, out: Optional[torch.Tensor] = None,
+               out_scale: float = 1.0) -> torch.Tensor:
+        """``u`` columns [c0, ..) hold q | k | v | gate -> the gated heads [T, heads vdim] (see ``GatedAttention.attend``)."""
+        s = self.spec
+        rope = _shared_rope(self._rope, (s.rot_dims, s.rot_base, None), meta.max_keys, u.device)
+        return seqmix.decay_linear_attention(u, c0, self.decay, run.ssm, meta, s.heads, s.dim, s.vdim, self.eps, s.act, rope,
+                                             s.rot_dims, s.k_scale, self.norm_w, s.norm, s.gate_act, out, out_scale)
+
+    def forward(self, h: torch.Tensor, meta: seqmix.RaggedMeta, run) -> torch.Tensor:
+        return self.o(self.attend(self.proj_in(h), 0, meta, run))
+
+
+class AttentionRetention(nn.Module):
+    """Gated attention and linear attention with fixed decays side by side on one input, left_scale and right_scale
+    times their outputs added.  One fused GEMM over the input produces both sides' q | k | v | gate; the scales are
+    applied in fp32 where each side's gate is, to heads that lie side by side in one row, so one output GEMM over
+    [W_o left | W_o right] adds the sides up."""
+
+    def __init__(self, spec: LayerSpec, width: int, eps: float, dtype, device):
+        super().__init__()
+        self.left = GatedAttention(spec.gated_attn, width, eps, dtype, device, inner=True)
+        self.right = DecayLinearAttention(spec.decay_attn, width, eps, dtype, device, inner=True)
+        self.scales = (spec.left_scale, spec.right_scale)
+        a, r = spec.gated_attn, spec.decay_attn
+        self.cols = (sum(a.proj_sizes), a.heads * a.vdim, r.heads * r.vdim)
+        self.proj_in = Linear(width, self.cols[0] + sum(r.in_sizes), False, dtype, device)
+        self.o = Linear(self.cols[1] + self.cols[2], width, False, dtype, device)
+
+    def forward(self, h: torch.Tensor, meta: seqmix.RaggedMeta, run) -> torch.Tensor:
+        u = self.proj_in(h)
+        c0, nl, nr = self.cols
+        y = torch.empty(h.shape[0], nl + nr, dtype=h.dtype, device=h.device)
+        self.left.attend(u, 0, meta, run, y[:, :nl], self.scales[0])
+        self.right.attend(u, c0, meta, run, y[:, nl:], self.scales[1])
+        return self.o(y)
 
 
 class GatedLinearAttention(nn.Module):

@@ -66,9 +66,9 @@ class MoEFeedForward(nn.Module):
         return shared, parts, wts
 
     def run(self, h: torch.Tensor) -> MoEOut:
-        """The squared-ReLU form with a grouped choice: h [T, W] -> MoEOut."""
+        """The form with a grouped choice (squared-ReLU or silu-gated experts): h [T, W] -> MoEOut."""
         s = self.spec
-        assert s.act == "relu2" and s.router == "softmax" and s.weight_on == "output"
+        assert s.router == "softmax" and s.weight_on == "output" and (s.act == "relu2" or (s.act == "silu_glu" and not s.shared_ff))
         idx, wts, shared_w = seqmix.moe_route_grouped(h, self.router, s.top, s.scale, self.correction, s.groups, s.groups_keep,
                                                       s.shared_gate)
         if s.shared_ff and h.shape[0] < seqmix.MOE_GEMM_MIN:

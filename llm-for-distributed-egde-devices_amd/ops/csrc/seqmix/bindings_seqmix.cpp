@@ -35,14 +35,16 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
                       const float* vb, const int* tok_seq, const int* tok_pos, const int* seq_slot, const int* ptab,
                       int ptab_ld, void* out, int rows, int H, int G, int D, int Dv, int page, int PB, float scale,
                       int window, int pool, int f32, int nsplit, float* part, int kld, int vld, int chunked, float cap,
-                      const float* slopes, const float* sink, int gate_elem, int keep_first, hipStream_t st);
+                      const float* slopes, const float* sink, int gate_elem, int keep_first, const float* rel, int rel_n,
+                      int out_ld, float out_scale, hipStream_t st);
 size_t edge_sm_attention_part_floats(int rows, int H, int G, int D, int Dv, int nsplit);
 int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const void* kp, const void* vp,
                            const float* kb, const float* vb, const int* seq_slot, const int* seq_start,
                            const int* seq_len, const int* seq_off, const int* ptab, int ptab_ld, void* out, int n,
                            int qtiles, int H, int G, int D, int Dv, int page, int PB, float scale, int window,
                            int pool, int kld, int vld, int chunked, float cap, const float* slopes, const float* sink,
-                           int gate_elem, int keep_first, hipStream_t st);
+                           int gate_elem, int keep_first, const float* rel, int rel_n, int out_ld, float out_scale,
+                           hipStream_t st);
 int edge_sm_conv_silu(const void* u, int ld, int c0, int C, const float* w, const float* bias, void* state,
                       const int* tok_seq, const int* tok_pos, const int* seq_slot, const int* seq_start,
                       const int* seq_len, const int* seq_off, void* out, int rows, int n, int taps, int f32,
@@ -84,14 +86,23 @@ int edge_sm_moe_route(const void* h, int W, const float* router, const float* bi
 int edge_sm_hyper_read_norm(const float* X, const float* in_w, const float* w, void* y, int rows, int S, int W, float eps,
                             int f32, hipStream_t st);
 int edge_sm_hyper_update(float* X, const float* mix, const float* out_w, const void* y, const void* parts, const float* pw,
-                         int K, int rows, int S, int W, const float* in2, const float* w2, void* h, float eps, int f32,
-                         hipStream_t st);
+                         const int* part_rows, int part_total, int K, int rows, int S, int W, const float* in2,
+                         const float* w2, void* h, float eps, int f32, hipStream_t st);
 int edge_sm_poly_norm(const void* z, int ld, const float* coef, void* y, int rows, int F, float eps, int f32,
                       hipStream_t st);
 int edge_sm_qk_norm_rope_write(const void* proj, int ld, const int* tok_seq, const int* tok_pos, const int* seq_slot,
                                const int* ptab, int ptab_ld, const float* qw, const float* kw, float eps, const float* cs,
                                const float* vcs, const float* temp, void* q_out, void* kp, void* vp, int rows, int H, int G,
-                               int D, int Dv, int rot, int page, int f32, hipStream_t st);
+                               int D, int Dv, int rot, int page, const float* bias, float qt_coef, int qt_every, int f32,
+                               hipStream_t st);
+int edge_sm_decay_fused(int P);
+int edge_sm_decay_step_ok(int N);
+int edge_sm_decay_attn(const void* u, int ld, const float* dec, const float* cs, int rot, float k_scale, int silu,
+                       const float* norm_w, int all_heads, int gate_silu, float* state, const int* seq_slot,
+                       const int* seq_start, const int* seq_len, const int* seq_off, void* out, int out_ld, float out_scale,
+                       float* y, float* sloc, int rows, int n, int max_chunks, int H, int N, int P, float eps, int f32,
+                       hipStream_t st);
+int edge_sm_softcap(const void* z, float* out, long n, float cap, int f32, hipStream_t st);
 int edge_sm_unrotate_gate(const void* a, const void* gate, int gate_ld, const int* tok_pos, const float* vcs, void* out,
                           int rows, int HD, int Dv, int f32, hipStream_t st);
 int edge_sm_moe_experts(const void* h, int W, const int* idx, int top, const void* w_gu, const void* w_down, int ff,
@@ -294,9 +305,10 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
                         const std::optional<at::Tensor>& seq_start, const std::optional<at::Tensor>& seq_len,
                         const std::optional<at::Tensor>& seq_off, int64_t n, int64_t qtiles, bool chunked, double softcap,
                         const std::optional<at::Tensor>& slopes, const std::optional<at::Tensor>& sink,
-                        int64_t keep_first) {
-  // chunked: `window` is a chunk size and the gate is [T, H * Dv] (see attn_kernel); keep_first: the first
-  // tokens of a sequence that stay visible behind a sliding window
+                        int64_t keep_first, const std::optional<at::Tensor>& rel, const std::optional<at::Tensor>& dst,
+                        double out_scale) {
+  // chunked: `window` is a chunk size (see attn_kernel); keep_first: the first tokens of a sequence that stay visible
+  // behind a sliding window; rel [H, n]: a number per distance added to the scores; dst: where the result goes
   TORCH_CHECK(keep_first >= 0 && (keep_first == 0 || (window > 0 && !chunked)), "keep_first goes with a sliding window");
   chk_i32(tok_seq, "tok_seq");
   chk_i32(tok_pos, "tok_pos");
@@ -316,9 +328,16 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
   int gate_ld = 0, PB = 0;
   if (gate) {
     gate_ld = row_ld(*gate, "gate");
-    TORCH_CHECK(gate->size(0) == T && gate->size(1) == (chunked ? H * Dv : H) && gate->scalar_type() == q.scalar_type(),
-                "gate: [T, H] (one per head) or [T, H Dv] (one per coordinate)");
+    TORCH_CHECK(gate->size(0) == T && (gate->size(1) == H * Dv || (!chunked && gate->size(1) == H)) &&
+                    gate->scalar_type() == q.scalar_type(), "gate: [T, H] (one per head) or [T, H Dv] (one per coordinate)");
   }
+  const float* rel_p = nullptr;
+  if (rel) {
+    chk_f32(*rel, "rel");
+    TORCH_CHECK(rel->dim() == 2 && rel->size(0) == H && rel->size(1) >= 1 && pool == 0, "rel: fp32 [H, distances], no pooled blocks");
+    rel_p = rel->data_ptr<float>();
+  }
+  const int rel_n = rel ? (int)rel->size(1) : 0;
   const float* slopes_p = nullptr;
   const float* sink_p = nullptr;
   if (slopes) {
@@ -332,7 +351,7 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
     sink_p = sink->data_ptr<float>();
   }
   TORCH_CHECK(!chunked || pool == 0, "chunked attention has no pooled blocks");
-  const int gate_elem = chunked && gate ? 1 : 0;
+  const int gate_elem = gate && gate->size(1) == H * Dv ? 1 : 0;
   if (pool > 0 && window > 0) {
     TORCH_CHECK(kb && vb, "pooled entries missing");
     chk_f32(*kb, "k_pool");
@@ -342,7 +361,11 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
                     vb->size(1) == PB && vb->size(3) == Dv, "pooled entries: [pages, ceil(page / pool), G, D]");
   }
   c10::hip::HIPGuardMasqueradingAsCUDA guard(q.device());
-  auto out = at::empty({T, H * Dv}, q.options());
+  if (dst)
+    TORCH_CHECK(row_ld(*dst, "out") >= H * Dv && dst->size(0) == T && dst->size(1) == H * Dv && dst->scalar_type() == q.scalar_type(),
+                "out: [T, H Dv] in q's dtype");
+  auto out = dst ? *dst : at::empty({T, H * Dv}, q.options());
+  const int out_ld = (int)out.stride(0);
   if (qtiles > 0 && q.scalar_type() == at::kBFloat16) {
     // prompt portions in bf16 (qtiles = sum of ceil(len / 64)): the MFMA kernel when it takes the head sizes
     TORCH_CHECK(seq_start && seq_len && seq_off, "sequence metadata missing");
@@ -358,7 +381,7 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
                                           ptab.data_ptr<int>(), (int)ptab.stride(0), out.data_ptr(), (int)n, (int)qtiles,
                                           (int)H, (int)G, (int)D, (int)Dv, (int)page, PB, (float)scale, (int)window,
                                           PB ? (int)pool : 0, (int)kld, (int)vld, chunked ? 1 : 0, (float)softcap, slopes_p,
-                                          sink_p, gate_elem, (int)keep_first, stream());
+                                          sink_p, gate_elem, (int)keep_first, rel_p, rel_n, out_ld, (float)out_scale, stream());
     if (rc != 1) {
       check(rc, "sm_attention_mfma");
       return out;
@@ -381,7 +404,8 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
                           ptab.data_ptr<int>(), (int)ptab.stride(0), out.data_ptr(), (int)T, (int)H, (int)G, (int)D, (int)Dv,
                           (int)page, PB, (float)scale, (int)window, PB ? (int)pool : 0, f32(q), nsplit,
                           nsplit > 1 ? part.data_ptr<float>() : nullptr, (int)kld, (int)vld, chunked ? 1 : 0, (float)softcap,
-                          slopes_p, sink_p, gate_elem, (int)keep_first, stream()), "sm_attention");
+                          slopes_p, sink_p, gate_elem, (int)keep_first, rel_p, rel_n, out_ld, (float)out_scale, stream()),
+        "sm_attention");
   return out;
 }
 
@@ -807,6 +831,7 @@ at::Tensor sm_hyper_read_norm(const at::Tensor& X, const std::optional<at::Tenso
 std::optional<at::Tensor> sm_hyper_update(at::Tensor& X, const std::optional<at::Tensor>& mix,
                                           const std::optional<at::Tensor>& out_w, const std::optional<at::Tensor>& y,
                                           const std::optional<at::Tensor>& parts, const std::optional<at::Tensor>& part_w,
+                                          const std::optional<at::Tensor>& part_rows,
                                           const std::optional<at::Tensor>& next_in, const std::optional<at::Tensor>& next_w,
                                           double eps) {
   chk_f32(X, "X");
@@ -832,6 +857,10 @@ std::optional<at::Tensor> sm_hyper_update(at::Tensor& X, const std::optional<at:
       chk_f32(*part_w, "part_w");
       TORCH_CHECK(part_w->numel() == T * K, "part_w: fp32 [T, K]");
     }
+    if (part_rows) {
+      chk_i32(*part_rows, "part_rows");
+      TORCH_CHECK(part_rows->numel() == T * K, "part_rows: int32 [T, K]");
+    }
   }
   c10::hip::HIPGuardMasqueradingAsCUDA guard(X.device());
   std::optional<at::Tensor> h;
@@ -846,8 +875,8 @@ std::optional<at::Tensor> sm_hyper_update(at::Tensor& X, const std::optional<at:
   }
   check(edge_sm_hyper_update(X.data_ptr<float>(), mix ? mix->data_ptr<float>() : nullptr,
                              out_w ? out_w->data_ptr<float>() : nullptr, y ? y->data_ptr() : nullptr,
-                             parts ? parts->data_ptr() : nullptr, parts && part_w ? part_w->data_ptr<float>() : nullptr, K,
-                             (int)T, (int)S, (int)W, (h && next_in) ? next_in->data_ptr<float>() : nullptr,
+                             parts ? parts->data_ptr() : nullptr, parts && part_w ? part_w->data_ptr<float>() : nullptr,
+                             parts && part_rows ? part_rows->data_ptr<int>() : nullptr, (int)T * K, K, (int)T, (int)S, (int)W, (h && next_in) ? next_in->data_ptr<float>() : nullptr,
                              h ? next_w->data_ptr<float>() : nullptr, h ? h->data_ptr() : nullptr, (float)eps, is_f32,
                              stream()), "sm_hyper_update");
   return h;
@@ -869,7 +898,8 @@ at::Tensor sm_qk_norm_rope_write(const at::Tensor& proj, const at::Tensor& tok_s
                                  const at::Tensor& seq_slot, const at::Tensor& ptab, const std::optional<at::Tensor>& qw,
                                  const std::optional<at::Tensor>& kw, double eps, const std::optional<at::Tensor>& rope,
                                  const std::optional<at::Tensor>& vrope, const std::optional<at::Tensor>& temp,
-                                 at::Tensor& kp, at::Tensor& vp, int64_t H, int64_t rot) {
+                                 at::Tensor& kp, at::Tensor& vp, int64_t H, int64_t rot,
+                                 const std::optional<at::Tensor>& bias, double qt_coef, int64_t qt_every) {
   const int ld = row_ld(proj, "proj");
   chk_i32(tok_seq, "tok_seq");
   chk_i32(tok_pos, "tok_pos");
@@ -903,7 +933,8 @@ at::Tensor sm_qk_norm_rope_write(const at::Tensor& proj, const at::Tensor& tok_s
                                    seq_slot.data_ptr<int>(), ptab.data_ptr<int>(), (int)ptab.stride(0), vec(qw, D, "q norm"),
                                    vec(kw, D, "k norm"), (float)eps, cs, vcs, vec(temp, H, "temp"), q.data_ptr(),
                                    kp.data_ptr(), vp.data_ptr(), (int)T, (int)H, (int)G, (int)D, (int)Dv, (int)rot, (int)page,
-                                   f32(proj), stream()), "sm_qk_norm_rope_write");
+                                   vec(bias, (H + G) * D + G * Dv, "bias"), (float)qt_coef, (int)qt_every, f32(proj), stream()),
+        "sm_qk_norm_rope_write");
   return q;
 }
 
@@ -1174,6 +1205,60 @@ at::Tensor sm_gla(const at::Tensor& u, const at::Tensor& a2, const at::Tensor& b
   return out;
 }
 
+// u columns [c0, c0 + 2 H N + 2 H P) = q | k | v | gate; dec fp32 [2, H] (decays, their log2); all_heads: the norm runs over
+// the heads together; chunks > 0: the form over 64-token chunks (chunks = sum of ceil(len / 64), max_chunks = the largest)
+at::Tensor sm_decay_attn(const at::Tensor& u, int64_t c0, const at::Tensor& dec, const std::optional<at::Tensor>& rope, int64_t rot,
+                         double k_scale, bool silu, const std::optional<at::Tensor>& norm_w, bool all_heads, bool gate_silu,
+                         at::Tensor& state, const at::Tensor& tok_pos, const at::Tensor& seq_slot, const at::Tensor& seq_start,
+                         const at::Tensor& seq_len, const at::Tensor& seq_off, int64_t n, int64_t H, int64_t N, int64_t P,
+                         double eps, const std::optional<at::Tensor>& dst, double out_scale, int64_t chunks, int64_t max_chunks) {
+  TORCH_CHECK(is_act(u), "u: fp32 / bf16");
+  const int ld = row_ld(u, "u");
+  chk_f32(dec, "decay");
+  chk_f32(state, "state");
+  for (const at::Tensor* t : {&tok_pos, &seq_slot, &seq_start, &seq_len, &seq_off}) chk_i32(*t, "metadata");
+  const int64_t T = u.size(0);
+  TORCH_CHECK(H > 0 && N > 0 && P > 0 && dec.numel() == 2 * H && c0 >= 0 && c0 + 2 * H * N + 2 * H * P <= u.size(1),
+              "u [T, .. q | k | v | gate ..], decay fp32 [2, H]");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == N && state.size(3) == P, "state: fp32 [slots, heads, N, P]");
+  TORCH_CHECK(tok_pos.numel() == T && seq_slot.numel() >= n && seq_start.numel() >= n && seq_len.numel() >= n && seq_off.numel() >= n,
+              "sequence metadata: [n]");
+  TORCH_CHECK(rot == 0 || (rope && rope->is_cuda() && rope->scalar_type() == at::kFloat && rope->is_contiguous() && rope->dim() == 3 &&
+                           rope->size(1) * 2 == rot && rope->size(2) == 2), "rope: fp32 [pos, rot / 2, 2]");
+  if (norm_w) {
+    chk_f32(*norm_w, "norm weight");
+    TORCH_CHECK(norm_w->numel() == (all_heads ? H * P : P), "norm weight: fp32 [P] or [H P]");
+  }
+  if (dst)
+    TORCH_CHECK(row_ld(*dst, "out") >= H * P && dst->size(0) == T && dst->size(1) == H * P && dst->scalar_type() == u.scalar_type(),
+                "out: [T, H P] in u's dtype");
+  TORCH_CHECK(chunks > 0 || edge_sm_decay_step_ok((int)N), "key channels per head: the token-by-token form takes up to 256");
+  TORCH_CHECK(chunks == 0 || (chunks * 64 >= T && max_chunks > 0 && max_chunks <= chunks), "chunk counts do not cover the step");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(u.device());
+  auto out = dst ? *dst : at::empty({T, H * P}, u.options());
+  auto f = u.options().dtype(at::kFloat);
+  at::Tensor y, sloc;
+  if (all_heads || !edge_sm_decay_fused((int)P)) y = at::empty({T, H * P}, f);
+  if (chunks > 0) sloc = at::empty({chunks, H, N, P}, f);
+  const size_t col = (size_t)c0 * u.element_size();
+  check(edge_sm_decay_attn((const char*)u.data_ptr() + col, ld, dec.data_ptr<float>(), rot > 0 ? rope->data_ptr<float>() : nullptr,
+                           (int)rot, (float)k_scale, silu, norm_w ? norm_w->data_ptr<float>() : nullptr, all_heads, gate_silu,
+                           state.data_ptr<float>(), seq_slot.data_ptr<int>(), seq_start.data_ptr<int>(), seq_len.data_ptr<int>(),
+                           seq_off.data_ptr<int>(), out.data_ptr(), (int)out.stride(0), (float)out_scale,
+                           y.defined() ? y.data_ptr<float>() : nullptr, sloc.defined() ? sloc.data_ptr<float>() : nullptr, (int)T,
+                           (int)n, chunks > 0 ? (int)max_chunks : 0, (int)H, (int)N, (int)P, (float)eps, f32(u), stream()),
+        "sm_decay_attn");
+  return out;
+}
+
+at::Tensor sm_softcap(const at::Tensor& z, double cap) {
+  TORCH_CHECK(z.is_cuda() && is_act(z) && z.is_contiguous(), "z: fp32 / bf16, contiguous");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(z.device());
+  auto out = at::empty(z.sizes(), z.options().dtype(at::kFloat));
+  check(edge_sm_softcap(z.data_ptr(), out.data_ptr<float>(), (long)z.numel(), (float)cap, f32(z), stream()), "sm_softcap");
+  return out;
+}
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -1218,4 +1303,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("sm_head_expand_gate", &sm_head_expand_gate);
   m.def("sm_heads_gate", &sm_heads_gate);
   m.def("sm_gla", &sm_gla);
+  m.def("sm_decay_attn", &sm_decay_attn);
+  m.def("sm_softcap", &sm_softcap);
 }

@@ -26,12 +26,10 @@ constexpr float LOG2E = 1.4426950408889634f;
 __device__ __forceinline__ float log_sigmoid(float z) {
   return z >= 0.f ? -log1pf(expf(-z)) : z - log1pf(expf(z));
 }
-__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
 // log2 sigmoid(z) = -(max(-z, 0) log2 e + log2(1 + 2^{-|z| log2 e}))
 __device__ __forceinline__ float log2_sigmoid(float z) {
   return -(fmaxf(-z, 0.f) * LOG2E + __builtin_amdgcn_logf(1.f + ex2(-fabsf(z) * LOG2E)));
 }
-__device__ __forceinline__ v4f mfma4(float a, float b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
 // ---------------------------------------------------------------------------------- token by token
 // One workgroup of NW waves per (sequence, head, 64 CG value columns): lane = column, wave w keeps the state rows

@@ -56,14 +56,16 @@ __global__ void __launch_bounds__(NT) hyper_read_norm_kernel(const float* __rest
 
 // X [rows, S, W] fp32 in place: X[t, r] <- sum_s mix[s, r] X[t, s] + out_w[r] v, v = y[t] + sum_k pw[t, k] parts[t, k]
 // (fp32, k order; y / parts / pw may be null; pw null with parts: ones).  mix null: X[t, r] += v.
+// rows given: choice k of token t sits at row rows[t, k] (of nrows) of parts, else at t K + k.
 // C = columns per thread and pass (4 with 16-byte stream accesses when W % 4 == 0, else 1).
 // NEXT: the next sublayer's read and norm in the same pass (one workgroup per token, dynamic LDS u [W]):
 // h[t] = u / sqrt(mean(u^2) + eps) * w2 with u = sum_r in2[r] X_new[t, r] (in2 null: the plain sum).
 template <typename T, int C, bool NEXT>
 __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X, const float* __restrict__ mix,
                                                           const float* __restrict__ out_w, const T* __restrict__ y,
-                                                          const T* __restrict__ parts, const float* __restrict__ pw, int K,
-                                                          int S, int W, const float* __restrict__ in2,
+                                                          const T* __restrict__ parts, const float* __restrict__ pw,
+                                                          const int* __restrict__ rows, int nrows, int K, int S, int W,
+                                                          const float* __restrict__ in2,
                                                           const float* __restrict__ w2, T* __restrict__ h, float eps) {
   extern __shared__ __attribute__((aligned(16))) float u_s[];
   __shared__ float m_s[MAXS * MAXS + MAXS];
@@ -94,9 +96,11 @@ __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X,
 #pragma unroll
     for (int i = 0; i < C; ++i) v[i] = 0.f;
     if (y) ld4(y + t * W + c, v);
+#pragma unroll 4
     for (int k = 0; k < K; ++k) {
       float p[C];
-      ld4(parts + (t * K + k) * W + c, p);
+      const size_t pr = rows ? (size_t)min(max(rows[t * K + k], 0), nrows - 1) : t * K + k;
+      ld4(parts + pr * W + c, p);
       const float wk = pw ? pw[t * K + k] : 1.f;
 #pragma unroll
       for (int i = 0; i < C; ++i) v[i] += wk * p[i];
@@ -205,9 +209,14 @@ __global__ void __launch_bounds__(NT) poly_norm_kernel(const T* __restrict__ z, 
   }
 }
 
-// proj row = q [H, D] | k [G, D] | v [G, Dv] | ...  One wave per head at a time.  q / k: divided by the head's
-// root mean square times qw / kw (null: no norm), pairs (2i, 2i + 1), i < rot / 2, turned by cs[pos, i] =
-// (cos, sin), q times temp[h] (null: 1).  v: pairs over all Dv turned by vcs[pos, m] (null: copied).  q goes
+// q's factor at a position: 1 + coef ln(floor((pos + 1) / every) + 1) (every 0: 1)
+__device__ __forceinline__ float pos_temp(int pos, float coef, int every) {
+  return every > 0 ? 1.f + coef * logf((float)((pos + 1) / every + 1)) : 1.f;
+}
+
+// proj row = q [H, D] | k [G, D] | v [G, Dv] | ...  One wave per head at a time.  bias (q | k | v; null: 0) is added, then
+// q / k: divided by the head's root mean square times qw / kw (null: no norm), pairs (2i, 2i + 1), i < rot / 2, turned by
+// cs[pos, i] = (cos, sin), q times temp[h] (null: 1) and pos_temp.  v: pairs over all Dv turned by vcs[pos, m] (null: copied).  q goes
 // to q_out [rows, H, D], k and v to the token's page row.
 template <typename T>
 __global__ void __launch_bounds__(NT) qk_norm_rope_write_kernel(
@@ -215,7 +224,7 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_kernel(
     const int* __restrict__ seq_slot, const int* __restrict__ ptab, int ptab_ld, const float* __restrict__ qw,
     const float* __restrict__ kw, float eps, const float* __restrict__ cs, const float* __restrict__ vcs,
     const float* __restrict__ temp, T* __restrict__ q_out, T* __restrict__ kp, T* __restrict__ vp, int H, int G, int D,
-    int Dv, int rot, int page) {
+    int Dv, int rot, int page, const float* __restrict__ bias, float qt_coef, int qt_every) {
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int pos = tok_pos[t], slot = seq_slot[tok_seq[t]];
   const size_t prow = (size_t)ptab[(size_t)slot * ptab_ld + pos / page] * page + pos % page;
@@ -226,19 +235,21 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_kernel(
     if (unit < H + G) {
       const bool isq = unit < H;
       const T* src = row + (size_t)unit * D;
+      const float* b = bias ? bias + (size_t)unit * D : nullptr;
+      auto at = [&](int d) { return ldf<T>(src + d) + (b ? b[d] : 0.f); };
       const float* w = isq ? qw : kw;
       float r = 1.f;
       if (w) {
         float ss = 0.f;
-        for (int d = lane; d < D; d += 64) { const float v = ldf<T>(src + d); ss += v * v; }
+        for (int d = lane; d < D; d += 64) { const float v = at(d); ss += v * v; }
         r = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
       }
-      const float mul = (isq && temp) ? temp[unit] : 1.f;
+      const float mul = isq ? (temp ? temp[unit] : 1.f) * pos_temp(pos, qt_coef, qt_every) : 1.f;
       T* dst = isq ? q_out + ((size_t)t * H + unit) * D : kp + (prow * G + (unit - H)) * D;
       for (int d = lane; d < D; d += 64) {
-        float v = ldf<T>(src + d) * r * (w ? w[d] : 1.f);
+        float v = at(d) * r * (w ? w[d] : 1.f);
         if (c && d < rot) {
-          const float o = ldf<T>(src + (d ^ 1)) * r * (w ? w[d ^ 1] : 1.f);
+          const float o = at(d ^ 1) * r * (w ? w[d ^ 1] : 1.f);
           const float co = c[d & ~1], si = c[(d & ~1) + 1];
           v = (d & 1) ? v * co + o * si : v * co - o * si;
         }
@@ -247,11 +258,13 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_kernel(
     } else {
       const int g = unit - H - G;
       const T* src = row + (size_t)(H + G) * D + (size_t)g * Dv;
+      const float* b = bias ? bias + (size_t)(H + G) * D + (size_t)g * Dv : nullptr;
+      auto at = [&](int d) { return ldf<T>(src + d) + (b ? b[d] : 0.f); };
       T* dst = vp + (prow * G + g) * Dv;
       for (int d = lane; d < Dv; d += 64) {
-        float v = ldf<T>(src + d);
+        float v = at(d);
         if (cv) {
-          const float o = ldf<T>(src + (d ^ 1)), co = cv[d & ~1], si = cv[(d & ~1) + 1];
+          const float o = at(d ^ 1), co = cv[d & ~1], si = cv[(d & ~1) + 1];
           v = (d & 1) ? v * co + o * si : v * co - o * si;
         }
         stf<T>(dst + d, v);
@@ -270,7 +283,7 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_vec_kernel(
     const int* __restrict__ seq_slot, const int* __restrict__ ptab, int ptab_ld, const float* __restrict__ qw,
     const float* __restrict__ kw, float eps, const float* __restrict__ cs, const float* __restrict__ vcs,
     const float* __restrict__ temp, T* __restrict__ q_out, T* __restrict__ kp, T* __restrict__ vp, int H, int G, int D,
-    int Dv, int rot, int page, int LPH) {
+    int Dv, int rot, int page, int LPH, const float* __restrict__ bias, float qt_coef, int qt_every) {
   __shared__ float part_s[NT];
   const int t = blockIdx.x, tid = threadIdx.x;
   const int unit = blockIdx.y * (NT / LPH) + tid / LPH, d = (tid % LPH) * 8;
@@ -281,7 +294,12 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_vec_kernel(
   float v[8];
   float ss = 0.f;
   if (live) {
-    load8<T>(proj + (size_t)t * ld + (isv ? (size_t)(H + G) * D + (size_t)(unit - H - G) * Dv : (size_t)unit * D) + d, v);
+    const size_t col = (isv ? (size_t)(H + G) * D + (size_t)(unit - H - G) * Dv : (size_t)unit * D) + d;
+    load8<T>(proj + (size_t)t * ld + col, v);
+    if (bias) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] += bias[col + i];
+    }
     if (w) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
@@ -312,8 +330,8 @@ __global__ void __launch_bounds__(NT) qk_norm_rope_write_vec_kernel(
       }
     }
   }
-  if (isq && temp) {
-    const float mul = temp[unit];
+  if (isq && (temp || qt_every > 0)) {
+    const float mul = (temp ? temp[unit] : 1.f) * pos_temp(pos, qt_coef, qt_every);
 #pragma unroll
     for (int i = 0; i < 8; ++i) v[i] *= mul;
   }
@@ -367,29 +385,29 @@ int edge_sm_hyper_read_norm(const float* X, const float* in_w, const float* w, v
 
 // w2 given: the next sublayer's input h [rows, W] = norm(sum_r in2[r] X_new[:, r]) w2 is written in the same pass
 int edge_sm_hyper_update(float* X, const float* mix, const float* out_w, const void* y, const void* parts, const float* pw,
-                         int K, int rows, int S, int W, const float* in2, const float* w2, void* h, float eps, int f32,
-                         hipStream_t st) {
+                         const int* part_rows, int part_total, int K, int rows, int S, int W, const float* in2,
+                         const float* w2, void* h, float eps, int f32, hipStream_t st) {
   if (rows == 0) return 0;
-  if (S < 1 || S > MAXS || (!y && K == 0) || (mix && !out_w) || (w2 && !h)) return -2;
+  if (S < 1 || S > MAXS || (!y && K == 0) || (mix && !out_w) || (w2 && !h) || (part_rows && part_total < 1)) return -2;
   const bool vec = W % 4 == 0 && (((uintptr_t)X | (uintptr_t)y | (uintptr_t)parts) & 15) == 0;
   if (w2) {
     if ((size_t)W * 4 > 60 * 1024) return -3;
     if (vec)
       SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 4, true>), dim3(rows), dim3(NT), (size_t)W * 4, st, X, mix, out_w,
-                                   (const T*)y, (const T*)parts, pw, K, S, W, in2, w2, (T*)h, eps));
+                                   (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, in2, w2, (T*)h, eps));
     else
       SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 1, true>), dim3(rows), dim3(NT), (size_t)W * 4, st, X, mix, out_w,
-                                   (const T*)y, (const T*)parts, pw, K, S, W, in2, w2, (T*)h, eps));
+                                   (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, in2, w2, (T*)h, eps));
     return (int)hipGetLastError();
   }
   const int per = NT * (vec ? 4 : 1);
   const int gy = rows >= 1024 ? 1 : (W + per - 1) / per < 8 ? (W + per - 1) / per : 8;
   if (vec)
     SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 4, false>), dim3(rows, gy), dim3(NT), 0, st, X, mix, out_w,
-                                 (const T*)y, (const T*)parts, pw, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
+                                 (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
   else
     SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 1, false>), dim3(rows, gy), dim3(NT), 0, st, X, mix, out_w,
-                                 (const T*)y, (const T*)parts, pw, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
+                                 (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
   return (int)hipGetLastError();
 }
 
@@ -409,19 +427,21 @@ int edge_sm_poly_norm(const void* z, int ld, const float* coef, void* y, int row
 int edge_sm_qk_norm_rope_write(const void* proj, int ld, const int* tok_seq, const int* tok_pos, const int* seq_slot,
                                const int* ptab, int ptab_ld, const float* qw, const float* kw, float eps, const float* cs,
                                const float* vcs, const float* temp, void* q_out, void* kp, void* vp, int rows, int H, int G,
-                               int D, int Dv, int rot, int page, int f32, hipStream_t st) {
+                               int D, int Dv, int rot, int page, const float* bias, float qt_coef, int qt_every, int f32,
+                               hipStream_t st) {
   if (rows == 0) return 0;
-  if (rot % 2 || rot > D || (rot > 0 && !cs) || (vcs && Dv % 2)) return -2;
+  if (rot % 2 || rot > D || (rot > 0 && !cs) || (vcs && Dv % 2) || qt_every < 0) return -2;
   const int lph = (D > Dv ? D : Dv) / 8;                      // threads per head
   if (D % 8 == 0 && Dv % 8 == 0 && ld % 8 == 0 && lph >= 1 && lph <= NT &&
       (((uintptr_t)proj | (uintptr_t)q_out | (uintptr_t)kp | (uintptr_t)vp) & 31) == 0)
     SM_T(f32, hipLaunchKernelGGL(qk_norm_rope_write_vec_kernel<T>, dim3(rows, (H + 2 * G + NT / lph - 1) / (NT / lph)), dim3(NT),
                                  0, st, (const T*)proj, ld, tok_seq, tok_pos, seq_slot, ptab, ptab_ld, qw, kw, eps,
-                                 rot > 0 ? cs : nullptr, vcs, temp, (T*)q_out, (T*)kp, (T*)vp, H, G, D, Dv, rot, page, lph));
+                                 rot > 0 ? cs : nullptr, vcs, temp, (T*)q_out, (T*)kp, (T*)vp, H, G, D, Dv, rot, page, lph, bias,
+                                 qt_coef, qt_every));
   else
     SM_T(f32, hipLaunchKernelGGL(qk_norm_rope_write_kernel<T>, dim3(rows), dim3(NT), 0, st, (const T*)proj, ld, tok_seq,
                                  tok_pos, seq_slot, ptab, ptab_ld, qw, kw, eps, rot > 0 ? cs : nullptr, vcs, temp, (T*)q_out,
-                                 (T*)kp, (T*)vp, H, G, D, Dv, rot, page));
+                                 (T*)kp, (T*)vp, H, G, D, Dv, rot, page, bias, qt_coef, qt_every));
   return (int)hipGetLastError();
 }
 

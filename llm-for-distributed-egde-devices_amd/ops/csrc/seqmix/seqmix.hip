@@ -11,6 +11,7 @@
 // order, and the recurrence steps token by token.
 #include "common.h"
 #include "seqmix/seqmix_common.h"
+#include "seqmix/attn_mfma.h"
 
 namespace {
 
@@ -199,15 +200,16 @@ __global__ void __launch_bounds__(NT) pool_kernel(const T* __restrict__ kp, cons
 // broadcast reads), (B) wave w keeps the running max / sum of heads w, w + 4, .. and turns the
 // chunk's scores into weights, (C) wave w accumulates weight x value over its quarter of the
 // chunk with lane = value coordinate (coalesced row reads).  Tokens of the window first, then the
-// pooled blocks (fp32 rows): one softmax over both.  A score may be capped (cap tanh(s / cap), cap > 0) and
-// lose slope[head] * dist, dist = the query's distance to this thread's key.
+// pooled blocks (fp32 rows): one softmax over both.  A score may be capped (cap tanh(s / cap), cap > 0),
+// lose slope[head] * dist and gain rel[head, min(dist, rel_n - 1)], dist = the query's distance to this thread's key.
 constexpr int KC = 256;
 
 template <typename KT, int RMAX, int DVL, bool VEC>
 __device__ __forceinline__ void attn_chunk(const KT* __restrict__ kbase, const KT* __restrict__ vbase, int cnt, int g,
                                            int kld, int vld, int D, int Dv, int R, const float* q_s, float* s_s, int* row_s,
                                            float* m_s, float* l_s, float* a_s, int rowidx, float (&acc)[RMAX][VEC ? 8 : DVL],
-                                           float cap = 0.f, const float* sl_s = nullptr, int dist = 0) {
+                                           float cap = 0.f, const float* sl_s = nullptr, int dist = 0,
+                                           const float* __restrict__ rel = nullptr, int rel_n = 0) {
   constexpr int AW = VEC ? 8 : DVL;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   // (A) scores
@@ -241,6 +243,12 @@ __device__ __forceinline__ void attn_chunk(const KT* __restrict__ kbase, const K
     if (sl_s) {
 #pragma unroll
       for (int r = 0; r < RMAX; ++r) a[r] -= sl_s[r] * (float)dist;
+    }
+    if (rel && tid < cnt) {
+      const float* rd = rel + min(max(dist, 0), rel_n - 1);
+#pragma unroll
+      for (int r = 0; r < RMAX; ++r)
+        if (r < R) a[r] += rd[(size_t)r * rel_n];
     }
 #pragma unroll
     for (int r = 0; r < RMAX; ++r) s_s[r * KC + tid] = tid < cnt ? a[r] : -INFINITY;
@@ -344,7 +352,9 @@ __global__ void __launch_bounds__(NT) attn_kernel(const T* __restrict__ q, const
                                                   int page, int PB, float scale, int window, int pool, int nsp, int nsplit,
                                                   float* __restrict__ part, int kld, int vld, int chunked, float cap,
                                                   const float* __restrict__ slopes, const float* __restrict__ sink,
-                                                  int gate_elem, int keep_first) {
+                                                  int gate_elem, int keep_first, const float* __restrict__ rel, int rel_n,
+                                                  int out_ld, float out_scale) {
+  // rel [H, rel_n]: a number per head and distance, added to the score (attn_chunk); out rows lie out_ld apart
   // keep_first: the tokens j < keep_first stay visible behind a sliding window
   // chunked: `window` is a chunk size (query i sees floor(i / window) * window .. i); cap / slopes: see attn_chunk;
   // sink: a number per query head that joins the softmax denominator (it enters as the first key split's
@@ -385,6 +395,7 @@ __global__ void __launch_bounds__(NT) attn_kernel(const T* __restrict__ q, const
 #pragma unroll
     for (int dl = 0; dl < AW; ++dl) acc[r][dl] = 0.f;
   __syncthreads();
+  const float* rel_h = rel ? rel + (size_t)hq0 * rel_n : nullptr;
   const int jlo = window > 0 ? (chunked ? (i / window) * window : max(0, i - window + 1)) : 0;
   const int nt = i - jlo + 1;
   const int nb = (!chunked && window > 0 && pool > 0 && i - window + 1 > 0) ? (i - window + 1) / pool : 0;
@@ -398,14 +409,14 @@ __global__ void __launch_bounds__(NT) attn_kernel(const T* __restrict__ q, const
     const int j = c0 + tid;
     const int rowidx = j < kf ? pt[j / page] * page + j % page : 0;
     attn_chunk<T, RMAX, DVL, VEC>(kp, vp, min(KC, kf - c0), g, kld, vld, D, Dv, R, q_s, s_s, row_s, m_s, l_s, a_s, rowidx, acc,
-                                  cap, slopes ? sl_s : nullptr, i - j);
+                                  cap, slopes ? sl_s : nullptr, i - j, rel_h, rel_n);
   }
   for (int c0 = 0; c0 < nt; c0 += KC, ++ci) {
     if (ci < ci0 || ci >= ci1) continue;
     const int j = jlo + c0 + tid;
     const int rowidx = c0 + tid < nt ? pt[j / page] * page + j % page : 0;
     attn_chunk<T, RMAX, DVL, VEC>(kp, vp, min(KC, nt - c0), g, kld, vld, D, Dv, R, q_s, s_s, row_s, m_s, l_s, a_s, rowidx, acc,
-                                  cap, slopes ? sl_s : nullptr, i - j);
+                                  cap, slopes ? sl_s : nullptr, i - j, rel_h, rel_n);
   }
   for (int c0 = 0; c0 < nb; c0 += KC, ++ci) {
     if (ci < ci0 || ci >= ci1) continue;
@@ -454,16 +465,15 @@ __global__ void __launch_bounds__(NT) attn_kernel(const T* __restrict__ q, const
     const int r = e / Dv, h = hq0 + r;
     float o = red[e] / l_s[r];
     if (gate) o *= sigmoidf_(ldf<T>(gate + (size_t)t * gate_ld + (gate_elem ? h * Dv + e % Dv : h)));
-    stf<T>(out + ((size_t)t * H + h) * Dv + e % Dv, o);
+    stf<T>(out + (size_t)t * out_ld + h * Dv + e % Dv, o * out_scale);
   }
 }
-
 
 // sums the key-split partial results of attn_kernel: out = sum_z e^{m_z - M} acc_z / sum_z e^{m_z - M} l_z
 template <typename T>
 __global__ void __launch_bounds__(NT) attn_merge_kernel(const float* __restrict__ part, const T* __restrict__ gate,
                                                         int gate_ld, T* __restrict__ out, int H, int G, int Dv, int nsp,
-                                                        int nsplit, int rmax, int gate_elem) {
+                                                        int nsplit, int rmax, int gate_elem, int out_ld, float out_scale) {
   const int t = blockIdx.x, g = blockIdx.y / nsp, r0 = (blockIdx.y % nsp) * rmax;
   const int R = min(rmax, H / G - r0), hq0 = g * (H / G) + r0, stride = rmax * (Dv + 2);
   const float* src = part + ((size_t)t * gridDim.y + blockIdx.y) * nsplit * stride;
@@ -480,275 +490,7 @@ __global__ void __launch_bounds__(NT) attn_merge_kernel(const float* __restrict_
     }
     float o = acc / l;
     if (gate) o *= sigmoidf_(ldf<T>(gate + (size_t)t * gate_ld + (gate_elem ? (hq0 + r) * Dv + e % Dv : hq0 + r)));
-    stf<T>(out + ((size_t)t * H + hq0 + r) * Dv + e % Dv, o);
-  }
-}
-
-// ---------------------------------------------------------------------------------- attention, bf16 MFMA
-// Prompt portions in bf16: 64 query rows of one (sequence, head) per workgroup, 16 per wave, on
-// v_mfma_f32_16x16x32_bf16.  A key tile is one page of the sequence (64 tokens, rows G * D apart) or
-// 64 pooled blocks (fp32 rows rounded to bf16 while staging); per tile S = Q K^T from a padded-row
-// LDS image of K, the mask (window / block-complete rule) and the online softmax in fp32 in the
-// log2 domain, P to per-wave LDS as bf16, O += P V with V fragments read transposed from the
-// row-major V tile.  Tiles wholly outside a workgroup's window are never visited.
-constexpr int MQ = 64, MK = 64;
-
-// RH query heads of one kv head per workgroup: a staged key / value tile serves all of them
-// (second launch bound: workgroups per CU the register budget must allow - four for 64-wide heads, so the
-// 1024 workgroups of a 4096-token, 16-head prompt are resident at once)
-// KVS: the value of a cached row is its first Dv numbers (a latent cache, or values that are the keys): the
-// staged key tile serves as the value tile, nothing is loaded twice
-// EXT: scores are capped (cap tanh(s / cap), cap > 0) and lose slopes[head] * distance; chunked: `window` is a
-// chunk size (a query sees its own chunk's start .. itself), else a sliding window beside the sequence's first
-// keep_first tokens; sink[head] joins the softmax denominator; the gate is [T, H * Dv], one per output coordinate
-struct AttnExt {
-  float scale, cap;
-  const float* slopes;
-  const float* sink;
-  int chunked, keep_first;
-};
-
-template <int DK, int DV, int RH, bool KVS, bool EXT = false>
-__global__ void __launch_bounds__(NT, (DV * RH <= 4 ? 4 : (DV * RH <= 8 ? 2 : 1))) attn_mfma_kernel(
-    const bf16_t* __restrict__ q, const bf16_t* __restrict__ gate, int gate_ld, const bf16_t* __restrict__ kp,
-    const bf16_t* __restrict__ vp, const float* __restrict__ kb, const float* __restrict__ vb,
-    const int* __restrict__ seq_slot, const int* __restrict__ seq_start, const int* __restrict__ seq_len,
-    const int* __restrict__ seq_off, const int* __restrict__ ptab, int ptab_ld, bf16_t* __restrict__ out, int n, int H,
-    int G, int PB, float scale_log2, int window, int pool, int kld, int vld, AttnExt ext = AttnExt{}) {
-  constexpr int D = 32 * DK, Dv = 16 * DV;
-  constexpr float LOG2E = 1.4426950408889634f;
-  constexpr int KS = D * 2 + 16, VS = KVS ? KS : Dv * 2 + 16, PS = MK * 2 + 16;      // LDS row strides in bytes
-  static_assert(!KVS || Dv <= D, "a value slice lies inside the key row");
-  __shared__ __attribute__((aligned(16))) char k_lds[MK * KS];
-  __shared__ __attribute__((aligned(16))) char v_own[KVS ? 16 : MK * VS];
-  char* const v_lds = KVS ? k_lds : v_own;
-  __shared__ __attribute__((aligned(16))) char p_all[4 * 16 * PS];
-  constexpr int NPID = 1024;
-  __shared__ int pid_s[NPID];                                // the sequence's first page ids (one global hop per tile less)
-  typedef __attribute__((address_space(3))) v4s lds_v4s;
-  int qt = blockIdx.x, s = 0;
-  for (; s < n; ++s) {
-    const int nq = (seq_len[s] + MQ - 1) / MQ;
-    if (qt < nq) break;
-    qt -= nq;
-  }
-  if (s == n) return;
-  const int h0 = blockIdx.y * RH, g = h0 / (H / G);
-  const int start = seq_start[s], len = seq_len[s], off = seq_off[s];
-  const int* pt = ptab + (size_t)seq_slot[s] * ptab_ld;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, c16 = lane & 15;
-  char* p_lds = p_all + wave * 16 * PS;
-  const int wq0 = qt * MQ + wave * 16;                       // this wave's first row inside the portion
-  v8s qf[RH][DK];
-  {
-    const int t = wq0 + c16;
-#pragma unroll
-    for (int r = 0; r < RH; ++r)
-#pragma unroll
-      for (int kk = 0; kk < DK; ++kk)
-        qf[r][kk] = t < len ? *reinterpret_cast<const v8s*>(q + ((size_t)(off + t) * H + h0 + r) * D + kk * 32 + 8 * g4)
-                            : v8s{0, 0, 0, 0, 0, 0, 0, 0};
-  }
-  v4f o[RH][DV];
-  float m_i[RH][4], l_i[RH][4];
-#pragma unroll
-  for (int r = 0; r < RH; ++r) {
-#pragma unroll
-    for (int i = 0; i < DV; ++i) o[r][i] = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int i = 0; i < 4; ++i) { m_i[r][i] = -INFINITY; l_i[r][i] = 0.f; }
-  }
-  // EXT: a score in the log2 domain is c1 - c2 / (2^(xs s) + 1) - sl2 (i - j)  (cap tanh(x / cap) written with one
-  // exp2 and one rcp; no cap: s scale_log2 - sl2 (i - j)); clo = first position of each row's chunk
-  float sl2[RH];
-  int clo[4];
-  const float c1 = ext.cap * LOG2E, c2 = 2.f * ext.cap * LOG2E, xs = ext.cap > 0.f ? ext.scale * 2.f * LOG2E / ext.cap : 0.f;
-#pragma unroll
-  for (int r = 0; r < RH; ++r) sl2[r] = 0.f;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) clo[i] = 0;
-  if constexpr (EXT) {
-    if (window > 0) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int qpos = start + wq0 + 4 * g4 + i;
-        clo[i] = ext.chunked ? (qpos / window) * window : max(0, qpos - window + 1);
-      }
-    }
-#pragma unroll
-    for (int r = 0; r < RH; ++r) {
-      if (ext.slopes) sl2[r] = ext.slopes[h0 + r] * LOG2E;
-      if (ext.sink) {                                        // the sink: a starting maximum with sum 1 and no value
-#pragma unroll
-        for (int i = 0; i < 4; ++i) { m_i[r][i] = ext.sink[h0 + r] * LOG2E; l_i[r][i] = 1.f; }
-      }
-    }
-  }
-  const int imin = start + qt * MQ, imax = start + min(len, qt * MQ + MQ) - 1;
-  const int jlo = window > 0 ? ((EXT && ext.chunked) ? (imin / window) * window : max(0, imin - window + 1)) : 0;
-  const int nbmax = (window > 0 && pool > 0 && imax - window + 1 > 0) ? (imax - window + 1) / pool : 0;
-  // the tiles that hold kept first tokens and lie wholly before the window's first tile come first
-  const int nfirst = (EXT && window > 0 && !ext.chunked) ? min((ext.keep_first + MK - 1) / MK, jlo / MK) : 0;
-  const int tok_tiles = nfirst + imax / MK - jlo / MK + 1, ntiles = tok_tiles + (nbmax + MK - 1) / MK;
-  auto tile_base = [&](int tile) {                           // first position (token tiles) / block (pooled tiles) of a tile
-    return tile < nfirst ? tile * MK : tile < tok_tiles ? (jlo / MK + tile - nfirst) * MK : (tile - tok_tiles) * MK;
-  };
-  for (int i = tid; i < min(imax / MK + 1, NPID); i += NT) pid_s[i] = pt[i];
-  __syncthreads();
-  auto page_of = [&](int idx) { return idx < NPID ? pid_s[idx] : pt[idx]; };
-
-  // a tile's rows travel global -> registers while the tile before it computes, registers -> LDS
-  // between the two barriers
-  static_assert(DV % 2 == 0, "value chunks per thread");
-  constexpr int KL = DK, VL = KVS ? 0 : DV / 2;              // 16-byte chunks per thread per tile
-  uint4 kreg[KL], vreg[VL > 0 ? VL : 1];
-  auto load_tile = [&](int tile) {
-    const bool tok = tile < tok_tiles;
-    const int base = tile_base(tile);
-    const size_t prow = tok ? (size_t)page_of(base / MK) * MK : 0;
-#pragma unroll
-    for (int i = 0; i < KL + VL; ++i) {
-      const bool isk = i < KL;
-      const int e = tid + (isk ? i : i - KL) * NT, cpr = isk ? D / 8 : Dv / 8;
-      const int r = e / cpr, c = e % cpr;
-      uint4 v = make_uint4(0, 0, 0, 0);
-      if (tok) {
-        v = isk ? *reinterpret_cast<const uint4*>(kp + (prow + r) * kld + g * D + c * 8)
-                : *reinterpret_cast<const uint4*>(vp + (prow + r) * vld + g * Dv + c * 8);
-      } else if (base + r < nbmax) {
-        const int p0 = (base + r) * pool;
-        const size_t row = ((size_t)page_of(p0 / MK) * PB + (p0 % MK) / pool) * G + g;
-        float f[8];
-        load8<float>(isk ? kb + row * D + c * 8 : vb + row * Dv + c * 8, f);
-        v = pack8(f);
-      }
-      if (isk) kreg[i] = v;
-      else vreg[VL > 0 ? i - KL : 0] = v;
-    }
-  };
-  auto store_tile = [&]() {
-#pragma unroll
-    for (int i = 0; i < KL; ++i) {
-      const int e = tid + i * NT;
-      *reinterpret_cast<uint4*>(k_lds + (e / (D / 8)) * KS + (e % (D / 8)) * 16) = kreg[i];
-    }
-#pragma unroll
-    for (int i = 0; i < VL; ++i) {
-      const int e = tid + i * NT;
-      *reinterpret_cast<uint4*>(v_lds + (e / (Dv / 8)) * VS + (e % (Dv / 8)) * 16) = vreg[i];
-    }
-  };
-  if (ntiles > 0) load_tile(0);
-  for (int tile = 0; tile < ntiles; ++tile) {
-    const bool tok = tile < tok_tiles;
-    const int base = tile_base(tile);
-    __syncthreads();                                         // every wave is done with the previous tile
-    store_tile();
-    __syncthreads();
-    if (tile + 1 < ntiles) load_tile(tile + 1);
-#pragma unroll
-    for (int r = 0; r < RH; ++r) {
-    v4f sc[4];
-#pragma unroll
-    for (int nt = 0; nt < 4; ++nt) {
-      sc[nt] = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int kk = 0; kk < DK; ++kk) {
-        const v8s kf = *reinterpret_cast<const v8s*>(k_lds + (nt * 16 + c16) * KS + (kk * 32 + 8 * g4) * 2);
-        sc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[r][kk], kf, sc[nt], 0, 0, 0);
-      }
-    }
-    // lane holds S[row = 4 g4 + i][key = 16 nt + c16]
-    float alpha[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int qpos = start + wq0 + 4 * g4 + i;
-      const int seen = (window > 0 && pool > 0 && qpos - window + 1 > 0) ? (qpos - window + 1) / pool : 0;
-      float mx = -INFINITY;
-#pragma unroll
-      for (int nt = 0; nt < 4; ++nt) {
-        const int key = base + nt * 16 + c16;
-        bool vis;
-        float v;
-        if constexpr (EXT) {
-          vis = key <= qpos && (key >= clo[i] || key < ext.keep_first);
-          const float bias = sl2[r] * (float)(qpos - key);
-          if (ext.cap > 0.f)                                 // 2^(xs s) = inf gives the cap itself, 0 gives -cap
-            v = c1 - c2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[nt][i] * xs) + 1.f) - bias;
-          else
-            v = sc[nt][i] * scale_log2 - bias;
-          v = vis ? v : -INFINITY;
-        } else {
-          vis = tok ? (key <= qpos && (window <= 0 || qpos - key < window)) : key < seen;
-          v = vis ? sc[nt][i] * scale_log2 : -INFINITY;
-        }
-        sc[nt][i] = v;
-        mx = fmaxf(mx, v);
-      }
-#pragma unroll
-      for (int o_ = 1; o_ < 16; o_ <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o_, 64));
-      const float mnew = fmaxf(m_i[r][i], mx);
-      const float msafe = (mnew == -INFINITY) ? 0.f : mnew;
-      alpha[i] = __builtin_amdgcn_exp2f(m_i[r][i] - msafe);
-      float rs = 0.f;
-#pragma unroll
-      for (int nt = 0; nt < 4; ++nt) {
-        const float p = __builtin_amdgcn_exp2f(sc[nt][i] - msafe);
-        sc[nt][i] = p;
-        rs += p;
-      }
-#pragma unroll
-      for (int o_ = 1; o_ < 16; o_ <<= 1) rs += __shfl_xor(rs, o_, 64);
-      l_i[r][i] = l_i[r][i] * alpha[i] + rs;
-      m_i[r][i] = mnew;
-    }
-#pragma unroll
-    for (int dt = 0; dt < DV; ++dt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) o[r][dt][i] *= alpha[i];
-#pragma unroll
-    for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        *reinterpret_cast<bf16_t*>(p_lds + (4 * g4 + i) * PS + (nt * 16 + c16) * 2) = f2bf(sc[nt][i]);
-    __builtin_amdgcn_s_waitcnt(0xC07F);                      // lgkmcnt(0): this wave's P rows are in LDS
-    __builtin_amdgcn_wave_barrier();
-#pragma unroll
-    for (int ks = 0; ks < 2; ++ks) {
-      const v8s pf = *reinterpret_cast<const v8s*>(p_lds + c16 * PS + (ks * 32 + 8 * g4) * 2);
-      const int key0 = ks * 32 + 8 * g4, qq = c16 >> 2, pp = c16 & 3;
-#pragma unroll
-      for (int dt = 0; dt < DV; ++dt) {
-        const char* a0 = v_lds + (key0 + qq) * VS + (dt * 16 + 4 * pp) * 2;
-        const v4s lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)(a0));
-        const v4s hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)(a0 + 4 * VS));
-        const v8s vf = v8s{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-        o[r][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf, vf, o[r][dt], 0, 0, 0);
-      }
-    }
-      __builtin_amdgcn_wave_barrier();                     // this wave's P reads precede the next head's P writes
-    }
-  }
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int t = wq0 + 4 * g4 + i;
-    if (t < len) {
-#pragma unroll
-      for (int r = 0; r < RH; ++r) {
-        float inv = l_i[r][i] > 0.f ? 1.f / l_i[r][i] : 0.f;
-        if constexpr (!EXT) {
-          if (gate) inv *= sigmoidf_(bf2f(gate[(size_t)(off + t) * gate_ld + h0 + r]));
-        }
-#pragma unroll
-        for (int dt = 0; dt < DV; ++dt) {
-          float ov = o[r][dt][i] * inv;
-          if constexpr (EXT) {
-            if (gate) ov *= sigmoidf_(bf2f(gate[(size_t)(off + t) * gate_ld + (h0 + r) * Dv + dt * 16 + c16]));
-          }
-          out[((size_t)(off + t) * H + h0 + r) * Dv + dt * 16 + c16] = f2bf(ov);
-        }
-      }
-    }
+    stf<T>(out + (size_t)t * out_ld + (hq0 + r) * Dv + e % Dv, o * out_scale);
   }
 }
 
@@ -1237,9 +979,11 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
                       const float* vb, const int* tok_seq, const int* tok_pos, const int* seq_slot, const int* ptab,
                       int ptab_ld, void* out, int rows, int H, int G, int D, int Dv, int page, int PB, float scale,
                       int window, int pool, int f32, int nsplit, float* part, int kld, int vld, int chunked, float cap,
-                      const float* slopes, const float* sink, int gate_elem, int keep_first, hipStream_t st) {
+                      const float* slopes, const float* sink, int gate_elem, int keep_first, const float* rel, int rel_n,
+                      int out_ld, float out_scale, hipStream_t st) {
   if (rows == 0) return 0;
-  if (G <= 0 || H % G || Dv > 512 || (chunked && pool > 0) || keep_first < 0) return -2;
+  if (G <= 0 || H % G || Dv > 512 || (chunked && pool > 0) || keep_first < 0 || (rel && (rel_n < 1 || pool > 0)) || out_ld < H * Dv)
+    return -2;
   const int R = H / G;
   const int rmax = edge_sm_attention_rmax(rows, H, G, D, Dv);
   if (rmax == 0) return -3;
@@ -1251,7 +995,7 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
   SM_T(f32, hipLaunchKernelGGL((attn_kernel<T, RM, DL, V>), dim3(rows, G * nsp, nsplit), dim3(NT), lds, st, (const T*)q,         \
                                (const T*)gate, gate_ld, (const T*)kp, (const T*)vp, kb, vb, tok_seq, tok_pos,       \
                                seq_slot, ptab, ptab_ld, (T*)out, H, G, D, Dv, page, PB, scale, window, pool, nsp, nsplit, part, \
-                               kld, vld, chunked, cap, slopes, sink, gate_elem, keep_first))
+                               kld, vld, chunked, cap, slopes, sink, gate_elem, keep_first, rel, rel_n, out_ld, out_scale))
 #define SM_ATT(RM, DL)               \
   do {                               \
     if (vec) SM_ATT_V(RM, DL, true); \
@@ -1274,7 +1018,7 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
 #undef SM_ATT_V
   if (nsplit > 1)
     SM_T(f32, hipLaunchKernelGGL(attn_merge_kernel<T>, dim3(rows, G * nsp), dim3(NT), 0, st, part, (const T*)gate, gate_ld,
-                                 (T*)out, H, G, Dv, nsp, nsplit, rmax, gate_elem));
+                                 (T*)out, H, G, Dv, nsp, nsplit, rmax, gate_elem, out_ld, out_scale));
   return (int)hipGetLastError();
 }
 
@@ -1339,6 +1083,12 @@ int edge_sm_ssd_chunked(const void* xbc, int Cx, const void* u, int ld, int dt0,
   return (int)hipGetLastError();
 }
 
+int edge_sm_attention_mfma_rel(const void* q, const void* gate, int gate_ld, const void* kp, const void* vp, const int* seq_slot,
+                               const int* seq_start, const int* seq_len, const int* seq_off, const int* ptab, int ptab_ld,
+                               void* out, int n, int qtiles, int H, int G, int D, int Dv, float scale, int window, int kld, int vld,
+                               const float* sink, int keep_first, const float* rel, int rel_n, int out_ld, float out_scale, int rh,
+                               hipStream_t st);
+
 // bf16 prompt portions on the matrix cores; returns 1 when no instantiation takes (D, Dv): the caller
 // then runs the general kernel
 int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const void* kp, const void* vp,
@@ -1346,7 +1096,8 @@ int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const v
                            const int* seq_len, const int* seq_off, const int* ptab, int ptab_ld, void* out, int n,
                            int qtiles, int H, int G, int D, int Dv, int page, int PB, float scale, int window,
                            int pool, int kld, int vld, int chunked, float cap, const float* slopes, const float* sink,
-                           int gate_elem, int keep_first, hipStream_t st) {
+                           int gate_elem, int keep_first, const float* rel, int rel_n, int out_ld, float out_scale,
+                           hipStream_t st) {
   if (page != MK || G <= 0 || H % G || kld % 8 || vld % 8) return 1;
   const bool extras = chunked || cap > 0.f || slopes || sink || gate_elem || keep_first > 0;
   if (n == 0 || qtiles == 0) return 0;
@@ -1361,16 +1112,24 @@ int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const v
   else if (R % 2 == 0 && (long)qtiles * (H / 2) >= 1024) rh = 2;
   const bool kvs = kp == vp && kld == vld;
   if (kvs && pool > 0) return 1;                             // pooled entries keep separate key / value rows
+  if (rel) {                                                 // a bias by distance: instantiations of its own (attn_rel.hip)
+    if (kvs || pool > 0 || chunked || cap > 0.f || slopes || (gate && !gate_elem)) return 1;
+    return edge_sm_attention_mfma_rel(q, gate, gate_ld, kp, vp, seq_slot, seq_start, seq_len, seq_off, ptab, ptab_ld, out, n,
+                                      qtiles, H, G, D, Dv, scale, window, kld, vld, sink, window > 0 ? keep_first : 0, rel, rel_n,
+                                      out_ld, out_scale, rh, st);
+  }
   if (extras) {
     // the capped / biased / chunked / sink / kept-first-tokens form: an element-wise gate or none, no pooled blocks
     if ((kvs && D != Dv) || pool > 0 || (gate && !gate_elem)) return 1;
-    const AttnExt ext{scale, cap, slopes, sink, chunked, (chunked || window <= 0) ? 0 : keep_first};
+    AttnExt ext{};
+    ext.scale = scale; ext.cap = cap; ext.slopes = slopes; ext.sink = sink; ext.chunked = chunked;
+    ext.keep_first = (chunked || window <= 0) ? 0 : keep_first;
 #define SM_MFX_R(DK, DV, RH) SM_MFX_RK(DK, DV, RH, true)
 #define SM_MFX_RK(DK, DV, RH, KVS)                                                                                   \
   hipLaunchKernelGGL((attn_mfma_kernel<DK, DV, RH, KVS, true>), dim3(qtiles, H / RH), dim3(NT), 0, st,               \
                      (const bf16_t*)q, (const bf16_t*)gate, gate_ld, (const bf16_t*)kp, (const bf16_t*)vp, kb, vb,   \
                      seq_slot, seq_start, seq_len, seq_off, ptab, ptab_ld, (bf16_t*)out, n, H, G, PB, sl2, window,   \
-                     pool, kld, vld, ext)
+                     pool, kld, vld, out_ld, out_scale, ext)
 #define SM_MFX(DK, DV)                    \
   do {                                    \
     if (rh == 4) SM_MFX_R(DK, DV, 4);     \
@@ -1406,7 +1165,8 @@ int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const v
   }
 #define SM_MF_ARGS                                                                                                  \
   dim3(NT), 0, st, (const bf16_t*)q, (const bf16_t*)gate, gate_ld, (const bf16_t*)kp, (const bf16_t*)vp, kb, vb,     \
-      seq_slot, seq_start, seq_len, seq_off, ptab, ptab_ld, (bf16_t*)out, n, H, G, PB, sl2, window, pool, kld, vld
+      seq_slot, seq_start, seq_len, seq_off, ptab, ptab_ld, (bf16_t*)out, n, H, G, PB, sl2, window, pool, kld, vld,  \
+      out_ld, out_scale
 #define SM_MF_R(DK, DV, RH, KVS) \
   hipLaunchKernelGGL((attn_mfma_kernel<DK, DV, RH, KVS>), dim3(qtiles, H / RH), SM_MF_ARGS)
 #define SM_MF(DK, DV)                             \

@@ -33,6 +33,9 @@ template <> __device__ __forceinline__ void store8<bf16_t>(bf16_t* p, const floa
 __device__ __forceinline__ float sigmoidf_(float x) { return 1.f / (1.f + expf(-x)); }
 __device__ __forceinline__ float siluf_(float x) { return x * sigmoidf_(x); }
 
+__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ v4f mfma4(float a, float b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
 constexpr int NT = 256;
 
 // sum over the 16 lanes of a DPP row (quad swaps, then row rotations by 4 and 8); every lane gets the sum

@@ -240,14 +240,18 @@ ATTN_MFMA_MIN = int(__import__("os").environ.get("EDGELLM_ATTN_MFMA_MIN", "16"))
 
 def window_pool_attention(q: torch.Tensor, gate: Optional[torch.Tensor], k_pages, v_pages, k_pool, v_pool,
                           meta: RaggedMeta, scale: float, window: Optional[int], pool: Optional[int],
-                          sink: Optional[torch.Tensor] = None, keep_first: int = 0) -> torch.Tensor:
+                          sink: Optional[torch.Tensor] = None, keep_first: int = 0, rel: Optional[torch.Tensor] = None,
+                          out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
     """q [T, H, D] -> [T, H * Dv].  Query position i sees the tokens j with 0 <= i - j < window and
     the pooled blocks b with b pool + pool - 1 <= i - window, in one softmax (fp32); head h's result
-    is multiplied by sigmoid(gate[t, h]) when ``gate`` ([T, H] view) is given.  ``keep_first``: the
-    tokens j < keep_first stay visible behind the window (j <= i).  ``sink`` (fp32 [H]): exp(sink[h])
-    joins head h's softmax denominator; it has no value."""
+    is multiplied by sigmoid(gate[t, h]) when ``gate`` is a [T, H] view, element by element when it is a
+    [T, H * Dv] view.  ``keep_first``: the tokens j < keep_first stay visible behind the window (j <= i).
+    ``sink`` (fp32 [H]): exp(sink[h]) joins head h's softmax denominator; it has no value.  ``rel`` (fp32
+    [H, n], from ``distance_bias_table``): rel[h, min(i - j, n - 1)] is added to the scaled score.  The result
+    times ``out_scale`` goes to ``out`` (a [T, H * Dv] view with dense rows in q's dtype) when it is given."""
     T, H, D = q.shape
     G, Dv = k_pages.shape[2], v_pages.shape[3]
+    assert rel is None or not pool, "pooled blocks have no distance"
     if _gpu(q):
         # bf16 steps with a portion of ATTN_MFMA_MIN tokens or more: the MFMA kernel (64 query rows per
         # workgroup); decode-sized steps and fp32: one workgroup per (token, kv head)
@@ -258,9 +262,9 @@ def window_pool_attention(q: torch.Tensor, gate: Optional[torch.Tensor], k_pages
                                    meta.tok_seq, meta.tok_pos, meta.seq_slot, meta.page_table, float(scale),
                                    int(window) if window is not None else 0, int(pool or 0), int(meta.max_keys),
                                    meta.seq_start, meta.seq_len, meta.seq_off, int(meta.n), int(qtiles), False, 0.0,
-                                   None, sink, int(keep_first if window is not None else 0))
+                                   None, sink, int(keep_first if window is not None else 0), rel, out, float(out_scale))
     page = meta.page
-    out = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
+    res = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
     R = H // G
     for slot, start, n, off in meta.host:
         L = start + n
@@ -272,6 +276,8 @@ def window_pool_attention(q: torch.Tensor, gate: Optional[torch.Tensor], k_pages
         i = torch.arange(start, L, device=q.device)
         s = torch.einsum("ngrd,lgd->ngrl", qi, k) * scale
         d = i[:, None] - pos[None]
+        if rel is not None:
+            s = s + rel[:, d.clamp(0, rel.shape[1] - 1)].view(G, R, n, L).permute(2, 0, 1, 3)
         vis = d >= 0
         if window is not None:
             vis &= (d < window) | (pos[None] < keep_first)
@@ -292,10 +298,29 @@ def window_pool_attention(q: torch.Tensor, gate: Optional[torch.Tensor], k_pages
         if sink is not None:
             s = torch.cat([s, sink.float().view(1, G, R, 1).expand(n, G, R, 1)], -1)
         p = torch.softmax(s, -1)[..., :vals.shape[0]]
-        out[off:off + n] = torch.einsum("ngrl,lgd->ngrd", p, vals).reshape(n, H, Dv)
+        res[off:off + n] = torch.einsum("ngrl,lgd->ngrd", p, vals).reshape(n, H, Dv)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())[..., None]
-    return out.reshape(T, H * Dv).to(q.dtype)
+        res = res * torch.sigmoid(gate.float()).view(T, H, -1)
+    return _into(out, (res * out_scale).reshape(T, H * Dv).to(q.dtype))
+
+
+def _into(out: Optional[torch.Tensor], res: torch.Tensor) -> torch.Tensor:
+    return res if out is None else out.copy_(res)
+
+
+def distance_bias_table(rel: torch.Tensor, far: int) -> torch.Tensor:
+    """rel [B, H] (a number per bucket of distances and head) -> fp32 [H, n]: the numbers by distance, up to the first
+    distance of the last bucket (every longer one shares its number).  Distances below B / 2 have a bucket each; the
+    others fall into B / 2 + floor(ln(d / (B / 2)) / ln(far / (B / 2)) (B - B / 2)), at most B - 1."""
+    import math
+    B, half = rel.shape[0], rel.shape[0] // 2
+    assert B >= 2 and far > half
+    idx, d = [], 0
+    while not idx or idx[-1] < B - 1:
+        # an edge that is exactly a whole number must not fall short of it by the logarithms' rounding
+        idx.append(d if d < half else min(B - 1, half + math.floor(math.log(d / half) / math.log(far / half) * (B - half) + 1e-9)))
+        d += 1
+    return rel.float()[torch.tensor(idx, device=rel.device)].t().contiguous()
 
 
 def distance_slopes(heads: int, device=None) -> torch.Tensor:
@@ -321,7 +346,7 @@ def chunk_attention(q: torch.Tensor, gate: Optional[torch.Tensor], k_pages: torc
         return _ext().sm_attention(q, gate, k_pages, k_pages, None, None, meta.tok_seq, meta.tok_pos, meta.seq_slot,
                                    meta.page_table, float(scale), int(chunk or 0), 0, int(meta.max_keys), meta.seq_start,
                                    meta.seq_len, meta.seq_off, int(meta.n), int(qtiles), True, float(softcap or 0.0),
-                                   slopes, sink, 0)
+                                   slopes, sink, 0, None, None, 1.0)
     page, R = meta.page, H // G
     out = torch.empty(T, H, D, dtype=torch.float32, device=q.device)
     for slot, start, n, off in meta.host:
@@ -654,6 +679,66 @@ def gated_linear_attention(u: torch.Tensor, a2: torch.Tensor, a2_b: torch.Tensor
     return head_norm_gate(y, u[:, 2 * HN + HP:2 * HN + 2 * HP], norm_w, heads, eps, u.dtype, act="silu")
 
 
+# --------------------------------------------------------------------------- linear attention with fixed decays
+DECAY_CHUNK_MIN = int(__import__("os").environ.get("EDGELLM_DECAY_CHUNK_MIN", "24"))
+
+
+def decay_table(decay, device=None) -> torch.Tensor:
+    """fp32 [2, H]: the heads' decays and their log2 (a decay of 0: a log so low that every power but the zeroth is 0)."""
+    import math
+    return torch.tensor([list(decay), [math.log2(d) if d > 0 else -1e4 for d in decay]], dtype=torch.float32, device=device)
+
+
+def decay_linear_attention(u: torch.Tensor, c0: int, decay: torch.Tensor, state: torch.Tensor, meta: RaggedMeta, heads: int,
+                           N: int, P: int, eps: float, act: str = "none", rope: Optional[torch.Tensor] = None,
+                           rot_dims: int = 0, k_scale: float = 1.0, norm_w: Optional[torch.Tensor] = None, norm: str = "head",
+                           gate_act: str = "silu", out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
+    """u columns [c0, ..) hold q [heads, N] | k [heads, N] | v [heads, P] | gate [heads, P] (a layer's fused input
+    projection) -> [T, heads P] in u's dtype.
+
+    In fp32, per head: ``act`` "silu": q, k and v through silu; q's and k's first ``rot_dims`` coordinates turned by
+    ``rope[pos, i]`` = (cos, sin), i paired with i + rot_dims / 2; k times ``k_scale``; S <- decay[0, h] S + k v^T;
+    o = S^T q.  ``norm`` "head": each head's o over its root mean square (times ``norm_w`` fp32 [P], None: 1); "all": the
+    heads together over theirs (``norm_w`` fp32 [heads P]).  Then times silu / sigmoid (``gate_act``) of the gate and
+    ``out_scale``, written to ``out`` (a [T, heads P] view with dense rows) when it is given.  ``decay`` from
+    ``decay_table``; state [slots, heads, N, P] fp32 is read (zero for a portion starting at 0) and left at the
+    portion's end."""
+    HN, HP = heads * N, heads * P
+    if _gpu(u):
+        # portions of DECAY_CHUNK_MIN tokens or more: kernels parallel over 64-token chunks; shorter steps (decode):
+        # one workgroup per (sequence, head), token by token
+        chunks = max_chunks = 0
+        if meta.max_len >= DECAY_CHUNK_MIN or N > 256:
+            per = [(h[2] + 63) // 64 for h in meta.host]
+            chunks, max_chunks = sum(per), max(per)
+        return _ext().sm_decay_attn(u, int(c0), decay, rope if rot_dims else None, int(rot_dims), float(k_scale),
+                                    act == "silu", norm_w, norm == "all", gate_act == "silu", state, meta.tok_pos,
+                                    meta.seq_slot, meta.seq_start, meta.seq_len, meta.seq_off, int(meta.n), int(heads), int(N),
+                                    int(P), float(eps), out, float(out_scale), int(chunks), int(max_chunks))
+    T = u.shape[0]
+    x = u[:, c0:c0 + 2 * HN + 2 * HP].float()
+    f = F.silu if act == "silu" else (lambda t: t)
+    q, k, v = f(x[:, :HN]).view(T, heads, N), f(x[:, HN:2 * HN]).view(T, heads, N), f(x[:, 2 * HN:2 * HN + HP]).view(T, heads, P)
+    if rot_dims:
+        cs = rope[meta.tok_pos.long()][:, None]
+        q, k = _rotate_half(q, cs, rot_dims), _rotate_half(k, cs, rot_dims)
+    k = k * k_scale
+    y = torch.empty(T, heads, P, dtype=torch.float32, device=u.device)
+    for slot, start, n, off in meta.host:
+        S = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
+        for t in range(off, off + n):
+            S.mul_(decay[0][:, None, None]).add_(k[t][:, :, None] * v[t][:, None, :])
+            y[t] = torch.bmm(q[t][:, None, :], S)[:, 0]
+        state[slot] = S
+    y = y.view(T, 1, HP) if norm == "all" else y
+    y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)
+    if norm_w is not None:
+        y = y * norm_w.float()
+    g = x[:, 2 * HN + HP:]
+    y = y.reshape(T, HP) * (F.silu(g) if gate_act == "silu" else torch.sigmoid(g)) * out_scale
+    return _into(out, y.to(u.dtype))
+
+
 # --------------------------------------------------------------------------- gated delta rule
 def delta_prepare(qkv: torch.Tensor, u: torch.Tensor, b0: int, a: torch.Tensor, dt_bias: torch.Tensor,
                   A_log: torch.Tensor, heads: int, kv_heads: int, N: int):
@@ -915,6 +1000,13 @@ def glu_gelu(u: torch.Tensor, ff: int) -> torch.Tensor:
     return (F.gelu(u[:, :ff].float(), approximate="tanh") * u[:, ff:2 * ff].float()).to(u.dtype)
 
 
+def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap tanh(z / cap) in fp32 (logits of any dtype in, fp32 out)."""
+    if _gpu(z):
+        return _ext().sm_softcap(z, float(cap))
+    return cap * torch.tanh(z.float() / cap)
+
+
 # --------------------------------------------------------------------------- residual streams
 def hyper_read_norm(X: torch.Tensor, in_w: Optional[torch.Tensor], weight: torch.Tensor, eps: float, out_dtype) -> torch.Tensor:
     """X fp32 [T, S, W] (S copies of the residual stream) -> RMS norm of u = sum_s in_w[s] X[:, s]
@@ -926,22 +1018,26 @@ def hyper_read_norm(X: torch.Tensor, in_w: Optional[torch.Tensor], weight: torch
 
 
 def hyper_update(X: torch.Tensor, mix: Optional[torch.Tensor], out_w: Optional[torch.Tensor], y: Optional[torch.Tensor],
-                 parts: Optional[torch.Tensor] = None, part_w: Optional[torch.Tensor] = None, nxt: Optional[tuple] = None):
+                 parts: Optional[torch.Tensor] = None, part_w: Optional[torch.Tensor] = None, nxt: Optional[tuple] = None,
+                 part_rows: Optional[torch.Tensor] = None):
     """X fp32 [T, S, W], in place, all streams at once from the old ones:
     X[:, r] <- sum_s mix[s, r] X[:, s] + out_w[r] v, with v = y + sum_k part_w[:, k] parts[:, k] summed in
     fp32 in k order (``y`` [T, W] or None; ``parts`` [T, K, W] with ``part_w`` fp32 [T, K]: a mixture's
-    expert outputs).  ``mix`` fp32 [S, S] indexed [from, to] and ``out_w`` fp32 [S]; both None: X += v.
+    expert outputs; ``part_rows`` int32 [T, K]: choice k of token t sits at that row of parts viewed [-1, W]; None:
+    at t K + k).  ``mix`` fp32 [S, S] indexed [from, to] and ``out_w`` fp32 [S]; both None: X += v.
     Returns X, or with ``nxt`` = (in_w, weight, eps) the next sublayer's input ``hyper_read_norm`` of the new
     streams in the dtype of y / parts, computed in the same pass."""
     if _gpu(X):
         if nxt is not None:
-            return _ext().sm_hyper_update(X, mix, out_w, y, parts, part_w, nxt[0], nxt[1], float(nxt[2]))
-        _ext().sm_hyper_update(X, mix, out_w, y, parts, part_w, None, None, 0.0)
+            return _ext().sm_hyper_update(X, mix, out_w, y, parts, part_w, part_rows, nxt[0], nxt[1], float(nxt[2]))
+        _ext().sm_hyper_update(X, mix, out_w, y, parts, part_w, part_rows, None, None, 0.0)
         return X
     if nxt is not None:
-        hyper_update(X, mix, out_w, y, parts, part_w)
+        hyper_update(X, mix, out_w, y, parts, part_w, None, part_rows)
         return hyper_read_norm(X, nxt[0], nxt[1], nxt[2], (y if y is not None else parts).dtype)
     v = y.float() if y is not None else torch.zeros_like(X[:, 0])
+    if parts is not None and part_rows is not None:
+        parts = parts.reshape(-1, X.shape[2])[part_rows.long()]
     if parts is not None:
         for k in range(parts.shape[1]):
             v = v + (parts[:, k].float() if part_w is None else part_w[:, k:k + 1] * parts[:, k].float())
@@ -966,20 +1062,25 @@ def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
 # --------------------------------------------------------------------------- gated attention
 def qk_norm_rope_write(proj: torch.Tensor, meta: RaggedMeta, q_w: Optional[torch.Tensor], k_w: Optional[torch.Tensor],
                        eps: float, rope: Optional[torch.Tensor], v_rope: Optional[torch.Tensor], temp: Optional[torch.Tensor],
-                       k_pages: torch.Tensor, v_pages: torch.Tensor, heads: int, rot_dims: int) -> torch.Tensor:
+                       k_pages: torch.Tensor, v_pages: torch.Tensor, heads: int, rot_dims: int,
+                       bias: Optional[torch.Tensor] = None, q_temp: Optional[tuple] = None) -> torch.Tensor:
     """proj [T, q | k | v | ...] -> q [T, heads, D]; keys and values go to their pages at each token's
-    position.  In fp32, per head: q and k are divided by their root mean square over D (eps inside the
-    root) times ``q_w`` / ``k_w`` (fp32 [D]; None: no norm), then the pairs (2i, 2i + 1), i < rot_dims / 2,
-    are turned by ``rope[pos, i]`` = (cos, sin); q is multiplied by ``temp[h]`` (fp32 [heads]; None: 1).
+    position.  In fp32, per head: ``bias`` (fp32, q | k | v; None: 0) is added, q and k are divided by their root mean
+    square over D (eps inside the root) times ``q_w`` / ``k_w`` (fp32 [D]; None: no norm), then the pairs (2i, 2i + 1),
+    i < rot_dims / 2, are turned by ``rope[pos, i]`` = (cos, sin); q is multiplied by ``temp[h]`` (fp32 [heads]; None:
+    1) and by 1 + coef ln(floor((pos + 1) / every) + 1) with ``q_temp`` = (coef, every) (None: 1).
     The values' pairs (2m, 2m + 1) over all Dv coordinates are turned by ``v_rope[pos, m]`` (None: stored
     as they are)."""
     G, D, Dv = k_pages.shape[2], k_pages.shape[3], v_pages.shape[3]
     if _gpu(proj):
         return _ext().sm_qk_norm_rope_write(proj, meta.tok_seq, meta.tok_pos, meta.seq_slot, meta.page_table, q_w, k_w,
                                             float(eps), rope if rot_dims else None, v_rope, temp, k_pages, v_pages,
-                                            int(heads), int(rot_dims))
+                                            int(heads), int(rot_dims), bias, float(q_temp[0]) if q_temp else 0.0,
+                                            int(q_temp[1]) if q_temp else 0)
     T = proj.shape[0]
-    x = proj.float()
+    x = proj[:, :(heads + G) * D + G * Dv].float()
+    if bias is not None:
+        x = x + bias.float()
     q = x[:, :heads * D].view(T, heads, D)
     k = x[:, heads * D:(heads + G) * D].view(T, G, D)
     v = x[:, (heads + G) * D:(heads + G) * D + G * Dv].view(T, G, Dv)
@@ -993,6 +1094,8 @@ def qk_norm_rope_write(proj: torch.Tensor, meta: RaggedMeta, q_w: Optional[torch
         q, k = _rotate_pairs(q, cs, rot_dims), _rotate_pairs(k, cs, rot_dims)
     if temp is not None:
         q = q * temp.float()[None, :, None]
+    if q_temp:
+        q = q * (1.0 + q_temp[0] * torch.log(((pos + 1) // q_temp[1] + 1).float()))[:, None, None]
     if v_rope is not None:
         v = _rotate_pairs(v, v_rope[pos][:, None], Dv)
     slot = meta.seq_slot.long()[meta.tok_seq.long()]
