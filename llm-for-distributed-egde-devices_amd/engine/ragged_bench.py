@@ -12,7 +12,11 @@ feed-forwards, two residual streams) beside the Vetevik model of equal width, he
 and active expert width; or (``--hybrid-family numizen``) the Numizen model (gated latent attention and
 gated linear attention beside a gelu-gated unit or group-limited squared-ReLU experts) beside the Pagonex
 model of equal width, heads, head sizes, latent ranks, state size and active feed-forward work, its latent
-attention without a window as well.
+attention without a window as well; or (``--hybrid-family felavik``) the Felavik model (gated attention with a
+distance bias side by side with retention, lightning attention, group-limited silu-gated experts) beside the
+Numizen model (the like recurrence and router) and the Fikupel model without window or kept tokens and with
+one residual stream (the like attention and layer form), both of equal width, heads, head and state sizes and
+active expert width.
 
 Sizes resemble real layers (random weights): the hybrid layer has windowed attention with pooled
 blocks + a Mamba-2 mixer + a squared-ReLU feed-forward; the comparison model is the
@@ -31,7 +35,7 @@ from typing import Dict, List
 
 import torch
 
-from ..models.configs import (ChunkAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, LatentAttnSpec, LayerSpec, ModelConfig, MoESpec,
+from ..models.configs import (ChunkAttnSpec, DecayAttnSpec, DeltaSpec, GatedAttnSpec, GLASpec, LatentAttnSpec, LayerSpec, ModelConfig, MoESpec,
                               SSDSpec, WindowAttnSpec, PRESETS)
 from ..models.decoder import build_model
 from ..models.hybrid import build_hybrid
@@ -132,6 +136,7 @@ FIKUPEL_SIZES = {
 
 
 def fikupel_config(s: dict) -> ModelConfig:
+    """``window`` None and ``keep`` 0: every earlier token is seen; ``streams`` 1: the plain residual sum."""
     moe = MoESpec(s["experts"], s["top"], 1.0, s["ff"], router="top_softmax", act="silu_glu", weight_on="output",
                   router_bias=True)
     llama3 = {"rope_type": "llama3", "factor": 8.0, "low_freq_factor": 1.0, "high_freq_factor": 4.0,
@@ -150,7 +155,8 @@ def fikupel_config(s: dict) -> ModelConfig:
     return ModelConfig(arch="fikupel", vocab_size=s["vocab"], hidden_size=s["width"], num_layers=s["layers"],
                        num_heads=s["heads"], num_kv_heads=s["kv"], intermediate_size=0, head_dim=s["dim"],
                        max_position_embeddings=1 << 20, norm="rms", norm_eps=1e-6, act="silu_glu", pos_emb="rope",
-                       tie_word_embeddings=True, name="fikupel-bench", layer_specs=specs, streams=s["streams"], hyper=True)
+                       tie_word_embeddings=True, name="fikupel-bench", layer_specs=specs, streams=s["streams"],
+                       hyper=s["streams"] > 1)
 
 
 # Numizen sizes: latent-attention and linear-attention layers alternate with the heads, ranks and state sizes of the
@@ -181,6 +187,36 @@ def numizen_config(s: dict) -> ModelConfig:
                        num_heads=s["heads"], num_kv_heads=1, intermediate_size=s["dense_ff"], head_dim=s["dim"],
                        max_position_embeddings=1 << 15, norm="dyt", norm_eps=1e-6, act="gelu_tanh", parallel_residual=True,
                        pos_emb="learned", name="numizen-bench", layer_specs=specs, layer_scale=True)
+
+
+# Felavik sizes: parallel (attention beside retention) and lightning layers alternate; heads, head sizes, state sizes and
+# experts as in the Fikupel / Numizen sizes of the same name, the active expert width as in Fikupel
+FELAVIK_SIZES = {
+    "w1024": dict(width=1024, layers=4, heads=16, kv=4, dim=64, vdim=64, buckets=32, far=512, r_heads=16, r_dim=64, r_vdim=64,
+                  experts=16, top=4, groups=4, keep=2, ff=1024, vocab=32000),
+    "w2048": dict(width=2048, layers=4, heads=16, kv=4, dim=128, vdim=128, buckets=32, far=1024, r_heads=16, r_dim=128,
+                  r_vdim=128, experts=32, top=4, groups=4, keep=2, ff=2048, vocab=32000),
+}
+
+
+def felavik_config(s: dict) -> ModelConfig:
+    moe = MoESpec(s["experts"], s["top"], 1.0, s["ff"], act="silu_glu", groups=s["groups"], groups_keep=s["keep"])
+    decay = tuple(1.0 - 2.0 ** (-2.0 - 8.0 * h / s["r_heads"]) for h in range(s["r_heads"]))
+    specs = []
+    for i in range(s["layers"]):
+        if i % 2 == 0:
+            a = GatedAttnSpec(s["heads"], s["kv"], s["dim"], s["vdim"], s["dim"] ** -0.5, rotate_values=False, temp=False, sink=False,
+                              qkv_bias=True, q_temp=(0.3, 1024), rel_buckets=s["buckets"], rel_max=s["far"])
+            r = DecayAttnSpec(s["r_heads"], s["r_dim"], s["r_vdim"], decay, rot_dims=s["r_dim"], rot_base=500000.0,
+                              k_scale=s["r_dim"] ** -0.5)
+            specs.append(LayerSpec("attention_retention", moe=moe, gated_attn=a, decay_attn=r, left_scale=0.7, right_scale=0.7))
+        else:
+            d = DecayAttnSpec(s["r_heads"], s["r_dim"], s["r_vdim"], decay, act="silu", norm="all", gate_act="sigmoid")
+            specs.append(LayerSpec("lightning", moe=moe, decay_attn=d))
+    return ModelConfig(arch="felavik", vocab_size=s["vocab"], hidden_size=s["width"], num_layers=s["layers"],
+                       num_heads=s["heads"], num_kv_heads=s["kv"], intermediate_size=0, head_dim=s["dim"],
+                       max_position_embeddings=1 << 20, norm="rms", norm_eps=1e-6, act="silu_glu", pos_emb="rope",
+                       name="felavik-bench", layer_specs=specs, streams=1, hyper=False, logit_softcap=30.0)
 
 
 def closest_config(s: dict) -> ModelConfig:
@@ -235,7 +271,7 @@ def op_times(eng: RaggedEngine, entries, close=()) -> Dict[str, float]:
              "group_rms_norm", "group_norm_residual", "chunk_attention", "delta_prepare_head", "glu_silu",
              "hyper_read_norm", "hyper_update", "poly_norm", "qk_norm_rope_write", "unrotate_gate",
              "embedding_learned", "parallel_update", "glu_gelu", "moe_route_grouped", "moe_experts_shared",
-             "latent_expand_write", "head_expand_gate", "gated_linear_attention"]
+             "latent_expand_write", "head_expand_gate", "gated_linear_attention", "decay_linear_attention", "softcap"]
     saved = {n: getattr(seqmix, n) for n in names}
     lin = F.linear
 
@@ -371,6 +407,25 @@ def run_numizen(sizes: List[str], prompt: int, batch: int, steps: int, device) -
             "decode_batch": batch, "decode_steps": steps, "sizes": res}
 
 
+def run_felavik(sizes: List[str], prompt: int, batch: int, steps: int, device) -> Dict:
+    res = {}
+    r2 = lambda d: {k: (round(v, 2) if isinstance(v, float) else v) for k, v in d.items()}
+    for name in sizes:
+        s, n, f = FELAVIK_SIZES[name], NUMIZEN_SIZES[name], dict(FIKUPEL_SIZES[name], window=None, keep=0, streams=1)
+        got = {}
+        for label, cfg, size in (("felavik", felavik_config(s), s), ("closest_numizen", numizen_config(n), n),
+                                 ("closest_fikupel", fikupel_config(f), f)):
+            got[label] = bench_hybrid(size, prompt, batch, steps, device, cfg)
+            torch.cuda.empty_cache()
+        res[name] = {"size": s, "closest_size": n, "closest_attention_size": f, **{k: r2(v) for k, v in got.items()}}
+        for k in ("numizen", "fikupel"):
+            for what in ("prefill", "decode"):
+                res[name][f"{what}_ratio_{k}"] = round(got["felavik"][f"{what}_tok_s"] / got[f"closest_{k}"][f"{what}_tok_s"], 3)
+    return {"metric": "prefill / decode tokens/s, Felavik layer-spec model vs the Numizen and Fikupel models of equal size",
+            "dtype": "bf16", "data": "synthetic (random weights, random prompt)", "prompt_tokens": prompt,
+            "decode_batch": batch, "decode_steps": steps, "sizes": res}
+
+
 def run(sizes: List[str], prompt: int = 4096, batch: int = 4, steps: int = 32, device=None, family: str = "nudadra") -> Dict:
     device = torch.device(device or "cuda:0")
     if family == "pagonex":
@@ -381,6 +436,8 @@ def run(sizes: List[str], prompt: int = 4096, batch: int = 4, steps: int = 32, d
         return run_fikupel(sizes, prompt, batch, steps, device)
     if family == "numizen":
         return run_numizen(sizes, prompt, batch, steps, device)
+    if family == "felavik":
+        return run_felavik(sizes, prompt, batch, steps, device)
     res = {}
     for name in sizes:
         s = SIZES[name]

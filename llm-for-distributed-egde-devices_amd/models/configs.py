@@ -1073,8 +1073,7 @@ def to_felavik_config(cfg: ModelConfig) -> dict:
             left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale, "bias_max": a.rel_max}
             if a.q_temp:
                 left["q_temp"] = {"coef": a.q_temp[0], "every": a.q_temp[1]}
-            if d.rot_dims:
-                m["rot"] = {"dims": d.rot_dims, "base": d.rot_base}
+            m["rot"] = {"dims": d.rot_dims, "base": d.rot_base}
             m = {"left": left, "right": m, "left_scale": s.left_scale, "right_scale": s.right_scale}
         mlp = None
         if s.moe is not None:
