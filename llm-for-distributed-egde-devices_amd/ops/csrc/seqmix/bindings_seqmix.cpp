@@ -37,6 +37,7 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
                       int window, int pool, int f32, int nsplit, float* part, int kld, int vld, int chunked, float cap,
                       const float* slopes, const float* sink, int gate_elem, int keep_first, const float* rel, int rel_n,
                       int out_ld, float out_scale, hipStream_t st);
+int edge_sm_attention_splits(int rows, int G, int chunks);
 size_t edge_sm_attention_part_floats(int rows, int H, int G, int D, int Dv, int nsplit);
 int edge_sm_attention_mfma(const void* q, const void* gate, int gate_ld, const void* kp, const void* vp,
                            const float* kb, const float* vb, const int* seq_slot, const int* seq_start,
@@ -391,8 +392,7 @@ at::Tensor sm_attention(const at::Tensor& q, const std::optional<at::Tensor>& ga
   int nsplit = 1;
   {
     const int64_t vis = (window > 0 ? std::min<int64_t>(window + keep_first, max_keys) : max_keys) + (PB ? max_keys / pool : 0);
-    const int64_t chunks = (vis + 255) / 256;
-    if (T * G <= 64 && chunks > 1) nsplit = (int)std::min<int64_t>(chunks, 8);
+    nsplit = edge_sm_attention_splits((int)T, (int)G, (int)((vis + 255) / 256));
   }
   at::Tensor part;
   if (nsplit > 1)

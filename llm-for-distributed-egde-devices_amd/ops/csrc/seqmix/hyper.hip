@@ -58,9 +58,10 @@ __global__ void __launch_bounds__(NT) hyper_read_norm_kernel(const float* __rest
 // (fp32, k order; y / parts / pw may be null; pw null with parts: ones).  mix null: X[t, r] += v.
 // rows given: choice k of token t sits at row rows[t, k] (of nrows) of parts, else at t K + k.
 // C = columns per thread and pass (4 with 16-byte stream accesses when W % 4 == 0, else 1).
+// MS: the most streams the instantiation holds (1: the plain residual sum in few registers).
 // NEXT: the next sublayer's read and norm in the same pass (one workgroup per token, dynamic LDS u [W]):
 // h[t] = u / sqrt(mean(u^2) + eps) * w2 with u = sum_r in2[r] X_new[t, r] (in2 null: the plain sum).
-template <typename T, int C, bool NEXT>
+template <typename T, int C, bool NEXT, int MS>
 __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X, const float* __restrict__ mix,
                                                           const float* __restrict__ out_w, const T* __restrict__ y,
                                                           const T* __restrict__ parts, const float* __restrict__ pw,
@@ -68,13 +69,13 @@ __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X,
                                                           const float* __restrict__ in2,
                                                           const float* __restrict__ w2, T* __restrict__ h, float eps) {
   extern __shared__ __attribute__((aligned(16))) float u_s[];
-  __shared__ float m_s[MAXS * MAXS + MAXS];
+  __shared__ float m_s[MS * MS + MS];
   __shared__ float red[NT / 64];
   const size_t t = blockIdx.x;
-  float a2[MAXS];
+  float a2[MS];
   float ss = 0.f;
 #pragma unroll
-  for (int s = 0; s < MAXS; ++s) a2[s] = (NEXT && s < S) ? (in2 ? in2[s] : 1.f) : 0.f;
+  for (int s = 0; s < MS; ++s) a2[s] = (NEXT && s < S) ? (in2 ? in2[s] : 1.f) : 0.f;
   if (mix) {
     for (int e = threadIdx.x; e < S * S + S; e += NT) m_s[e] = e < S * S ? mix[e] : out_w[e - S * S];
     __syncthreads();
@@ -105,9 +106,9 @@ __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X,
 #pragma unroll
       for (int i = 0; i < C; ++i) v[i] += wk * p[i];
     }
-    float xs[MAXS][C];
+    float xs[MS][C];
 #pragma unroll
-    for (int s = 0; s < MAXS; ++s) {
+    for (int s = 0; s < MS; ++s) {
       if (s < S) {
         if constexpr (C == 4) {
           const float4 a = *reinterpret_cast<const float4*>(xr + (size_t)s * W + c);
@@ -124,7 +125,7 @@ __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X,
 #pragma unroll
     for (int i = 0; i < C; ++i) u[i] = 0.f;
 #pragma unroll
-    for (int r = 0; r < MAXS; ++r) {
+    for (int r = 0; r < MS; ++r) {
       if (r < S) {
         float n[C];
 #pragma unroll
@@ -132,7 +133,7 @@ __global__ void __launch_bounds__(NT) hyper_update_kernel(float* __restrict__ X,
           if (mix) {
             float a = 0.f;
 #pragma unroll
-            for (int s = 0; s < MAXS; ++s)
+            for (int s = 0; s < MS; ++s)
               if (s < S) a += m_s[s * S + r] * xs[s][i];
             n[i] = a + m_s[S * S + r] * v[i];
           } else {
@@ -389,25 +390,28 @@ int edge_sm_hyper_update(float* X, const float* mix, const float* out_w, const v
                          const float* w2, void* h, float eps, int f32, hipStream_t st) {
   if (rows == 0) return 0;
   if (S < 1 || S > MAXS || (!y && K == 0) || (mix && !out_w) || (w2 && !h) || (part_rows && part_total < 1)) return -2;
+  if (w2 && (size_t)W * 4 > 60 * 1024) return -3;
   const bool vec = W % 4 == 0 && (((uintptr_t)X | (uintptr_t)y | (uintptr_t)parts) & 15) == 0;
-  if (w2) {
-    if ((size_t)W * 4 > 60 * 1024) return -3;
-    if (vec)
-      SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 4, true>), dim3(rows), dim3(NT), (size_t)W * 4, st, X, mix, out_w,
-                                   (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, in2, w2, (T*)h, eps));
-    else
-      SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 1, true>), dim3(rows), dim3(NT), (size_t)W * 4, st, X, mix, out_w,
-                                   (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, in2, w2, (T*)h, eps));
-    return (int)hipGetLastError();
-  }
   const int per = NT * (vec ? 4 : 1);
-  const int gy = rows >= 1024 ? 1 : (W + per - 1) / per < 8 ? (W + per - 1) / per : 8;
-  if (vec)
-    SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 4, false>), dim3(rows, gy), dim3(NT), 0, st, X, mix, out_w,
-                                 (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
-  else
-    SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, 1, false>), dim3(rows, gy), dim3(NT), 0, st, X, mix, out_w,
-                                 (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, nullptr, nullptr, (T*)nullptr, 0.f));
+  const int gy = w2 || rows >= 1024 ? 1 : (W + per - 1) / per < 8 ? (W + per - 1) / per : 8;
+#define SM_HU(C, NEXT, MS)                                                                                                   \
+  SM_T(f32, hipLaunchKernelGGL((hyper_update_kernel<T, C, NEXT, MS>), dim3(rows, gy), dim3(NT), NEXT ? (size_t)W * 4 : 0, st, \
+                               X, mix, out_w, (const T*)y, (const T*)parts, pw, part_rows, part_total, K, S, W, in2, w2,      \
+                               (T*)h, eps))
+#define SM_HUS(C, NEXT)                 \
+  do {                                  \
+    if (S == 1) SM_HU(C, NEXT, 1);      \
+    else SM_HU(C, NEXT, MAXS);          \
+  } while (0)
+  if (w2) {
+    if (vec) SM_HUS(4, true);
+    else SM_HUS(1, true);
+  } else {
+    if (vec) SM_HUS(4, false);
+    else SM_HUS(1, false);
+  }
+#undef SM_HUS
+#undef SM_HU
   return (int)hipGetLastError();
 }
 

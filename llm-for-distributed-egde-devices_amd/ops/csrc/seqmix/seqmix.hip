@@ -469,6 +469,8 @@ __global__ void __launch_bounds__(NT) attn_kernel(const T* __restrict__ q, const
   }
 }
 
+constexpr int MAX_SPLIT = 16;                                // workgroups that share a query's keys
+
 // sums the key-split partial results of attn_kernel: out = sum_z e^{m_z - M} acc_z / sum_z e^{m_z - M} l_z
 template <typename T>
 __global__ void __launch_bounds__(NT) attn_merge_kernel(const float* __restrict__ part, const T* __restrict__ gate,
@@ -479,14 +481,23 @@ __global__ void __launch_bounds__(NT) attn_merge_kernel(const float* __restrict_
   const float* src = part + ((size_t)t * gridDim.y + blockIdx.y) * nsplit * stride;
   for (int e = threadIdx.x; e < R * Dv; e += NT) {
     const int r = e / Dv;
+    float m[MAX_SPLIT], a[MAX_SPLIT], s[MAX_SPLIT];           // every split's numbers are in flight at once
+#pragma unroll
+    for (int z = 0; z < MAX_SPLIT; ++z) {
+      const float* p = src + min(z, nsplit - 1) * stride;
+      m[z] = p[rmax * Dv + r];
+      a[z] = p[e];
+      s[z] = p[rmax * Dv + rmax + r];
+    }
     float M = -INFINITY;
-    for (int z = 0; z < nsplit; ++z) M = fmaxf(M, src[z * stride + rmax * Dv + r]);
+#pragma unroll
+    for (int z = 0; z < MAX_SPLIT; ++z) M = fmaxf(M, m[z]);
     float acc = 0.f, l = 0.f;
-    for (int z = 0; z < nsplit; ++z) {
-      const float mz = src[z * stride + rmax * Dv + r];
-      const float wz = mz == -INFINITY ? 0.f : expf(mz - M);
-      acc += wz * src[z * stride + e];
-      l += wz * src[z * stride + rmax * Dv + rmax + r];
+#pragma unroll
+    for (int z = 0; z < MAX_SPLIT; ++z) {
+      const float wz = z >= nsplit || m[z] == -INFINITY ? 0.f : expf(m[z] - M);
+      acc += wz * a[z];
+      l += wz * s[z];
     }
     float o = acc / l;
     if (gate) o *= sigmoidf_(ldf<T>(gate + (size_t)t * gate_ld + (gate_elem ? (hq0 + r) * Dv + e % Dv : hq0 + r)));
@@ -970,6 +981,14 @@ int edge_sm_attention_rmax(int rows, int H, int G, int D, int Dv) {
   return attn_lds_bytes(rmax, D, Dv) > 64 * 1024 ? 0 : rmax;
 }
 
+// workgroups that share one query's keys (`chunks` runs of KC visible keys): more than one for few queries over many keys
+// (decode steps), as many as fill the chip
+int edge_sm_attention_splits(int rows, int G, int chunks) {
+  if (chunks <= 1 || (long)rows * G > 64) return 1;
+  const int want = max(8, 256 / (rows * G));
+  return min(min(chunks, want), MAX_SPLIT);
+}
+
 size_t edge_sm_attention_part_floats(int rows, int H, int G, int D, int Dv, int nsplit) {
   const int R = H / G, rmax = max(1, edge_sm_attention_rmax(rows, H, G, D, Dv)), nsp = (R + rmax - 1) / rmax;
   return (size_t)rows * G * nsp * nsplit * rmax * (Dv + 2);
@@ -988,7 +1007,7 @@ int edge_sm_attention(const void* q, const void* gate, int gate_ld, const void* 
   const int rmax = edge_sm_attention_rmax(rows, H, G, D, Dv);
   if (rmax == 0) return -3;
   const int nsp = (R + rmax - 1) / rmax;
-  if (nsplit < 1 || (nsplit > 1 && !part)) return -2;
+  if (nsplit < 1 || nsplit > MAX_SPLIT || (nsplit > 1 && !part)) return -2;
   const size_t lds = attn_lds_bytes(rmax, D, Dv);
   const bool vec = D % 8 == 0 && Dv % 8 == 0 && kld % 8 == 0 && vld % 8 == 0;
 #define SM_ATT_V(RM, DL, V)                                                                                         \

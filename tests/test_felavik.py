@@ -767,6 +767,38 @@ def test_bf16_attention_over_long_prompts(H, G, D, Dv, B, far, spike):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("H,G,D,Dv", [(64, 8, 64, 64), (32, 16, 64, 96), (64, 16, 128, 64)])
+def test_bf16_attention_with_heads_that_share_a_workgroup(H, G, D, Dv):
+    """Steps large enough for two or four heads per workgroup of the matrix-core kernel, gate and scale in its
+    epilogue, written beside other columns: sampled rows against float64."""
+    g = torch.Generator().manual_seed(H + Dv)
+    lens, dt = (3000, 1100), torch.bfloat16
+    cache = PagedCache([_Spec(gated_attn=GatedAttnSpec(H, G, D, Dv, 1.0))], 70, slots=2, page=64, dtype=dt, device="cuda")
+    slots = {s: cache.acquire() for s in range(2)}
+    meta = step_meta(cache, slots, [(0, 0, lens[0]), (1, 0, lens[1])], "cuda")
+    T = sum(lens)
+    assert sum((n + 63) // 64 for n in lens) * (H // (4 if (H // G) % 4 == 0 else 2)) >= 1024
+    rn = lambda *s: torch.randn(*s, generator=g).to(dt)
+    u, gate, rel = rn(T, (H + G) * D + G * Dv), rn(T, H * Dv), torch.randn(H, 300, generator=g) * 2
+    q = seqmix.qk_norm_rope_write(u.cuda(), meta, None, None, 1e-5, None, None, None, cache.run(0).k, cache.run(0).v, H, 0)
+    wide = torch.full((T, H * Dv + 24), 7.0, dtype=dt, device="cuda")
+    seqmix.window_pool_attention(q, gate.cuda(), cache.run(0).k, cache.run(0).v, None, None, meta, 0.1, None, None, None, 0, rel.cuda(),
+                                 wide[:, 8:8 + H * Dv], 0.5)
+    got = wide.cpu()
+    assert (got[:, :8] == 7).all() and (got[:, 8 + H * Dv:] == 7).all()
+    x, off = u.double(), 0
+    for n in lens:
+        k = x[off:off + n, H * D:(H + G) * D].view(n, G, D)
+        v = x[off:off + n, (H + G) * D:].view(n, G, Dv)
+        for i in (0, 63, 64, 301, 777, n - 1):
+            s = torch.einsum("grd,lgd->grl", x[off + i, :H * D].view(G, H // G, D), k[:i + 1]) * 0.1
+            s = s + rel.double()[:, (i - torch.arange(i + 1)).clamp(max=299)].view(G, H // G, i + 1)
+            o = torch.einsum("grl,lgd->grd", torch.softmax(s, -1), v[:i + 1]).reshape(-1) * torch.sigmoid(gate[off + i].double()) * 0.5
+            assert (got[off + i, 8:8 + H * Dv].double() - o).abs().max() < 2e-2 * max(1.0, o.abs().max().item()), (n, i)
+        off += n
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("precision", ["fp32", "bf16"])
 def test_sizes_that_are_not_multiples_of_eight(tmp_path, precision):
     """Odd widths and head sizes take the scalar kernel paths and unaligned slices of the fused projections."""
