@@ -178,7 +178,7 @@ class GatedAttnSpec:
     qkv_bias: bool = False
     q_temp: Optional[tuple] = None       # (coef, every)
     rel_buckets: int = 0
-    rel_max: int = 0
+    rel_max: float = 0
 
     @property
     def proj_sizes(self):
@@ -999,7 +999,7 @@ def from_felavik_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
     """The Felavik layout of ``config.json``: ``layers`` (``type`` = ``parallel`` or ``lightning``, ``mixer`` sizes and
     constants, ``mlp`` = mixture of experts or null, ``weights_of`` = the layer whose tensors serve this one),
     ``embedding.scale``, ``logit_softcap``, ``norm.eps``, ``vocab``, ``width``.  ``shapes`` (tensor name -> shape of
-    the checkpoint) supplies the number of distance buckets."""
+    the checkpoint) supplies the number of distance buckets (without it: ``rel_buckets`` of the entry, or 32)."""
     n, specs = len(c["layers"]), []
     for i, l in enumerate(c["layers"]):
         m, kind = l["mixer"], l["type"]
@@ -1022,7 +1022,7 @@ def from_felavik_config(c: dict, shapes: Optional[dict] = None) -> ModelConfig:
             ga = GatedAttnSpec(heads=int(a["heads"]), kv_heads=int(a.get("kv_heads", a["heads"])), dim=int(a["dim"]),
                                vdim=int(a["vdim"]), scale=float(a["scale"]), rotate_values=False, temp=False, sink=False,
                                qkv_bias=True, q_temp=(float(t["coef"]), int(t["every"])) if t else None,
-                               rel_buckets=buckets, rel_max=int(a["bias_max"]))
+                               rel_buckets=buckets, rel_max=a["bias_max"])
             if ga.heads % ga.kv_heads:
                 raise ValueError("heads must be a multiple of kv_heads")
             if buckets < 2 or ga.rel_max <= buckets // 2:
